@@ -98,9 +98,9 @@ int mi355_dense_grouped_ex(const void* x, int32_t ldx, int32_t M, const void* w,
                            const int32_t* offs, const int32_t* gather, const int32_t* tiles, int32_t max_tiles, const float* egate, int32_t ldg,
                            int32_t goff, mi355_stream_t stream);
 int mi355_hy_moe_route_ex(const float* z, int32_t ld, int32_t tokens, int32_t E, int32_t groups, int32_t keep, int32_t top, int32_t* ids, float* wts,
-                          int32_t score_sigmoid, int32_t group_top, float wscale, mi355_stream_t stream);
+                          int32_t score, int32_t group_top, float wscale, mi355_stream_t stream);
 int mi355_hy_moe_route_align_ex(const float* z, int32_t ld, int32_t tokens, int32_t E, int32_t groups, int32_t keep, int32_t top, int32_t* ids, float* wts,
-                                int32_t* offs, int32_t* src_row, int32_t* place_of, int32_t* tiles, int32_t score_sigmoid, int32_t group_top,
+                                int32_t* offs, int32_t* src_row, int32_t* place_of, int32_t* tiles, int32_t score, int32_t group_top,
                                 float wscale, mi355_stream_t stream);
 int mi355_hy_attn_prep_ex2(float* qkv, int32_t ld, int32_t koff, int32_t voff, const int32_t* geom, const float* kfreq, const float* vfreq,
                            int32_t v_norm, float eps, const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows,
@@ -118,6 +118,37 @@ int mi355_hy_chunk_plan(const int32_t* row_start, int32_t nseq, int32_t C, int32
                         int32_t* ones, mi355_stream_t stream);
 int mi355_hy_chunk_prefix(const int32_t* cs, const int32_t* sc, const int32_t* slot, const int32_t* first_pos, int32_t nseq, const float* decay, int32_t H,
                           int32_t per_head, float* chunk_state, float* state, mi355_stream_t stream);
+
+/* Parallel residual streams, a delta rule with a decay per key channel behind short convolutions, a matrix memory under exponential gates, attention with a
+ * gate per value channel, and a router whose weights are the softmax over the chosen logits (score 2 of the routing calls above). */
+int mi355_hy_streams(float* X, int32_t n, int32_t S, int32_t W, const float* a, float ca, const void* na, const float* b, float cb, const void* nb, float neps,
+                     const float* moe_y, const int32_t* moe_place, const float* moe_wts, int32_t moe_top, const float* mix, const float* wr, const float* rd,
+                     const int32_t* ids, const void* table, int32_t vocab, const int32_t* rows, const void* w, float eps, void* h, int32_t act_dtype,
+                     mi355_stream_t stream);
+int mi355_hy_short_conv(const float* proj, int32_t ld, int32_t rows, int32_t C, int32_t taps, const void* w, int32_t units, int32_t uq, int32_t dim,
+                        float qscale, float unit_eps, const float* hist, const int32_t* seq, const int32_t* row_start, const int32_t* slot,
+                        const int32_t* first_pos, float* out, int32_t lo, int32_t R, void* low, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_channel_delta_scan(const float* x, int32_t ld, int32_t ro, int32_t ko, int32_t vo, const float* z, int32_t ldz, const float* zbias,
+                                const float* rate, const float* bp, int32_t ldb, int32_t H, int32_t G, int32_t dim, int32_t vdim,
+                                const int32_t* row_start, const int32_t* slot, const int32_t* first_pos, int32_t nseq, float* state, float* out,
+                                const float* raw, int32_t ldr, int32_t C, int32_t taps, float* hist, mi355_stream_t stream);
+int mi355_hy_memory_scan(int32_t pass, const float* proj, int32_t ld, int32_t qo, int32_t ko, int32_t vo, int32_t io, int32_t fo, float cap, float qscale,
+                         float den_eps, int32_t H, int32_t dim, int32_t vdim, const int32_t* row_start, const int32_t* slot, const int32_t* first_pos,
+                         int32_t nseq, float* state, float* mstate, const float* gates, float* cdecay, float* den, float* out, mi355_stream_t stream);
+int mi355_hy_memory_gates(const float* proj, int32_t ld, int32_t io, int32_t fo, float cap, int32_t H, const int32_t* row_start, const int32_t* slot,
+                          const int32_t* first_pos, int32_t nseq, float* mstate, int32_t nz, float* out, mi355_stream_t stream);
+int mi355_hy_chunk_prefix_ex(const int32_t* cs, const int32_t* sc, const int32_t* slot, const int32_t* first_pos, int32_t nseq, const float* decay,
+                             const float* cdecay, int32_t H, int32_t per_head, float* chunk_state, float* state, mi355_stream_t stream);
+int mi355_hy_head_norm_ex2(const float* o, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg, int32_t goff,
+                           void* out, int32_t w_heads, int32_t gate_sigmoid, const float* den, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_attn_rows_ex2(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                           const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache, const void* vcache,
+                           void* out, int32_t splits, float* parts, int32_t window, float softcap, const float* ogate, int32_t ldg,
+                           int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_attn_tiles_ex2(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                            const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0, const int32_t* tile_n,
+                            int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, float softcap, const float* ogate,
+                            int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream);
 
 #ifdef __cplusplus
 }

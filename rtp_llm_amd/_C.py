@@ -197,6 +197,15 @@ HYBRID_SIGNATURES = {
     "mi355_hy_embed_scaled": (i32, [vp, i32, vp, i32, i32, f32, vp, vp, i32, vp]),
     "mi355_hy_chunk_plan": (i32, [vp, i32, i32, i32, vp, vp, vp, vp, vp, vp]),
     "mi355_hy_chunk_prefix": (i32, [vp, vp, vp, vp, i32, vp, i32, i32, vp, vp, vp]),
+    "mi355_hy_streams": (i32, [vp, i32, i32, i32, vp, f32, vp, vp, f32, vp, f32, vp, vp, vp, i32, vp, vp, vp, vp, vp, i32, vp, vp, f32, vp, i32, vp]),
+    "mi355_hy_short_conv": (i32, [vp, i32, i32, i32, i32, vp, i32, i32, i32, f32, f32, vp, vp, vp, vp, vp, vp, i32, i32, vp, i32, vp]),
+    "mi355_hy_channel_delta_scan": (i32, [vp, i32, i32, i32, i32, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, vp, vp]),
+    "mi355_hy_memory_scan": (i32, [i32, vp, i32, i32, i32, i32, i32, i32, f32, f32, f32, i32, i32, i32, vp, vp, vp, i32, vp, vp, vp, vp, vp, vp, vp]),
+    "mi355_hy_memory_gates": (i32, [vp, i32, i32, i32, f32, i32, vp, vp, vp, i32, vp, i32, vp, vp]),
+    "mi355_hy_chunk_prefix_ex": (i32, [vp, vp, vp, vp, i32, vp, vp, i32, i32, vp, vp, vp]),
+    "mi355_hy_head_norm_ex2": (i32, [vp, i32, i32, i32, vp, f32, vp, i32, i32, vp, i32, i32, vp, i32, vp]),
+    "mi355_hy_attn_rows_ex2": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, f32, vp, i32, i32, i32, vp]),
+    "mi355_hy_attn_tiles_ex2": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, f32, vp, i32, i32, i32, vp]),
     "mi355_hy_branch_norm": (i32, [vp, vp, f32, vp, f32, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, vp, i32, f32, vp, i32, vp]),
 }
 

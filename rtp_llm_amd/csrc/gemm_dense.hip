@@ -7,10 +7,10 @@
 //   * tile kernel, fp32:  64 x 64 block tile, 4 x 4 register micro-tiles, true fp32 FMAs (no reduced-precision matrix mode);
 //   * skinny kernel, bf16, 2 <= M <= 16: one block per 16 outputs, its waves split K, MFMA fragments loaded straight from memory;
 //   * row kernel (M = 1; fp32 up to M = 16): a wave per output column streams its weight row once, 16-byte loads, wave reduction at the end.
-//   * grouped forms of the tile kernels (per-head weights over column slices, or rows sorted by expert with a gather and a tile list) and
-//     of the row kernel (the few rows of a decode step, each with its own expert's weight): mi355_dense_grouped.
+//   * grouped forms of these kernels (per-head or per-branch weights over column slices; rows sorted by expert with a gather and a tile
+//     list; the few rows of a decode step, each with its own expert's weight): mi355_dense_grouped.
 // Epilogues: bias, gated activation act(gate) * up (weight rows grouped [32 gate | 32 up], so one lane holds both; also the clamped form
-// min(g, L) sigmoid(1.702 min(g, L)) (clamp(u, -L, L) + 1)), tanh soft cap.
+// min(g, L) sigmoid(1.702 min(g, L)) (clamp(u, -L, L) + 1)), an activation of the plain output (also the square of relu), tanh soft cap.
 // Output is fp32 or the activation type.  A result row depends only on its own input row: the k order of the accumulation is fixed by
 // the kernel, never by M or by the row's place in the batch.
 #include "common.h"
@@ -18,7 +18,7 @@
 
 namespace {
 
-constexpr int DN_ACT_NONE = 0, DN_ACT_RELU = 1, DN_ACT_SILU = 2, DN_ACT_GELU_TANH = 3, DN_ACT_TANH = 4, DN_ACT_SWIGLU_CLAMP = 5;
+constexpr int DN_ACT_NONE = 0, DN_ACT_RELU = 1, DN_ACT_SILU = 2, DN_ACT_GELU_TANH = 3, DN_ACT_TANH = 4, DN_ACT_SWIGLU_CLAMP = 5, DN_ACT_RELU2 = 6;
 
 struct DenseParams {
     const void* x; const void* w; const void* bias; void* y;
@@ -61,6 +61,7 @@ __device__ __forceinline__ float dn_act(float g, int act) {
     if (act == DN_ACT_SILU) return g / (1.f + __expf(-g));
     if (act == DN_ACT_GELU_TANH) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
     if (act == DN_ACT_TANH) return tanhf(g);
+    if (act == DN_ACT_RELU2) { const float r = g > 0.f ? g : 0.f; return r * r; }
     return g;
 }
 
@@ -298,16 +299,17 @@ __device__ __forceinline__ float dn_wave_sum(float v) {
 template <typename T, int MR, int NC, bool GATED>
 __global__ __launch_bounds__(256) void dense_rows_kernel(DenseParams p, int mbase) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int o0 = (blockIdx.x * 4 + wave) * NC;
+    const int o0 = (blockIdx.x * 4 + wave) * NC, grp = blockIdx.y;     // grp: group of a column-sliced launch (0 otherwise)
     const int nout = GATED ? p.N / 2 : p.N;
     if (o0 >= nout) return;
-    const T* X = (const T*)p.x;
+    const T* X = (const T*)p.x + p.xs * grp;
     const T* W0[NC];
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
         const int o = min(o0 + c, nout - 1);                       // a column past the end repeats the last one and is not stored
-        W0[c] = (const T*)p.w + (size_t)(GATED ? (o >> 5) * 64 + (o & 31) : o) * p.K;
+        W0[c] = (const T*)p.w + p.ws * grp + (size_t)(GATED ? (o >> 5) * 64 + (o & 31) : o) * p.K;
     }
+    const T* Bi = p.bias ? (const T*)p.bias + (size_t)grp * p.N : nullptr;
     const int rows = min(MR, p.M - mbase);
     float a0[MR][NC], a1[GATED ? MR : 1][NC];
 #pragma unroll
@@ -346,8 +348,8 @@ __global__ __launch_bounds__(256) void dense_rows_kernel(DenseParams p, int mbas
             const int o = o0 + c;
             if (lane != 0 || o >= nout) continue;
             const int n0 = GATED ? (o >> 5) * 64 + (o & 31) : o;
-            if (p.bias) { g += dn_ld((const T*)p.bias + n0); if (GATED) u += dn_ld((const T*)p.bias + n0 + 32); }
-            dn_store<T>(p, mbase + m, o, GATED ? dn_gated(g, u, p.act, p.act_param) : dn_act(g, p.act));
+            if (Bi) { g += dn_ld(Bi + n0); if (GATED) u += dn_ld(Bi + n0 + 32); }
+            dn_store<T>(p, mbase + m, (int)(p.ys * grp) + o, GATED ? dn_gated(g, u, p.act, p.act_param) : dn_act(g, p.act));
         }
     }
 }
@@ -406,10 +408,10 @@ void launch_rows(const DenseParams& p, hipStream_t st) {
     for (int mb = 0; mb < p.M; mb += 16) {
         const int r = p.M - mb;
         // few rows: one output per wave keeps the most waves streaming; more rows: several outputs per wave share the loads of x
-        if (r <= 2)      hipLaunchKernelGGL((dense_rows_kernel<T, 2, 1, GATED>), dim3((nout + 3) / 4), dim3(256), 0, st, p, mb);
-        else if (r <= 4) hipLaunchKernelGGL((dense_rows_kernel<T, 4, 2, GATED>), dim3((nout + 7) / 8), dim3(256), 0, st, p, mb);
-        else if (r <= 8) hipLaunchKernelGGL((dense_rows_kernel<T, 8, GATED ? 2 : 4, GATED>), dim3((nout + (GATED ? 7 : 15)) / (GATED ? 8 : 16)), dim3(256), 0, st, p, mb);
-        else             hipLaunchKernelGGL((dense_rows_kernel<T, 16, GATED ? 2 : 4, GATED>), dim3((nout + (GATED ? 7 : 15)) / (GATED ? 8 : 16)), dim3(256), 0, st, p, mb);
+        if (r <= 2)      hipLaunchKernelGGL((dense_rows_kernel<T, 2, 1, GATED>), dim3((nout + 3) / 4, p.G), dim3(256), 0, st, p, mb);
+        else if (r <= 4) hipLaunchKernelGGL((dense_rows_kernel<T, 4, 2, GATED>), dim3((nout + 7) / 8, p.G), dim3(256), 0, st, p, mb);
+        else if (r <= 8) hipLaunchKernelGGL((dense_rows_kernel<T, 8, GATED ? 2 : 4, GATED>), dim3((nout + (GATED ? 7 : 15)) / (GATED ? 8 : 16), p.G), dim3(256), 0, st, p, mb);
+        else             hipLaunchKernelGGL((dense_rows_kernel<T, 16, GATED ? 2 : 4, GATED>), dim3((nout + (GATED ? 7 : 15)) / (GATED ? 8 : 16), p.G), dim3(256), 0, st, p, mb);
     }
 }
 
@@ -422,13 +424,13 @@ template <bool GATED>
 __global__ __launch_bounds__(512) void dense_skinny_bf16_kernel(DenseParams p, int mbase) {
     __shared__ f32x4 red[8][2][64];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, NW = blockDim.x >> 6;
-    const int nout = GATED ? p.N / 2 : p.N;
+    const int nout = GATED ? p.N / 2 : p.N, grp = blockIdx.y;
     const int r = lane & 15, kq = (lane >> 4) * 8;
     const int o = min((int)blockIdx.x * 16 + r, nout - 1);
     const int n = GATED ? (o >> 5) * 64 + (o & 31) : o;
-    const bf16* wg = (const bf16*)p.w + (size_t)n * p.K + kq;
+    const bf16* wg = (const bf16*)p.w + p.ws * grp + (size_t)n * p.K + kq;
     const bf16* wu = wg + (size_t)32 * p.K;
-    const bf16* xr = (const bf16*)p.x + (size_t)min(mbase + r, p.M - 1) * p.ldx + kq;
+    const bf16* xr = (const bf16*)p.x + p.xs * grp + (size_t)min(mbase + r, p.M - 1) * p.ldx + kq;
     f32x4 ag = {0.f, 0.f, 0.f, 0.f}, au = {0.f, 0.f, 0.f, 0.f};
     const bf16x8 zero = {};
     const int stride = NW * 32;
@@ -465,8 +467,8 @@ __global__ __launch_bounds__(512) void dense_skinny_bf16_kernel(DenseParams p, i
         const int row = mbase + (lane >> 4) * 4 + e;
         if (row >= p.M) continue;
         float g = ag[e], u = au[e];
-        if (p.bias) { g += dn_ld((const bf16*)p.bias + nb); if (GATED) u += dn_ld((const bf16*)p.bias + nb + 32); }
-        dn_store<bf16>(p, row, oc, GATED ? dn_gated(g, u, p.act, p.act_param) : dn_act(g, p.act));
+        if (p.bias) { const bf16* Bi = (const bf16*)p.bias + (size_t)grp * p.N; g += dn_ld(Bi + nb); if (GATED) u += dn_ld(Bi + nb + 32); }
+        dn_store<bf16>(p, row, (int)(p.ys * grp) + oc, GATED ? dn_gated(g, u, p.act, p.act_param) : dn_act(g, p.act));
     }
 }
 
@@ -475,7 +477,7 @@ __global__ __launch_bounds__(512) void dense_skinny_bf16_kernel(DenseParams p, i
 // x [M, K] (row stride ldx) and w [N, K] of act_dtype (MI355_ACT_BF16 or MI355_ACT_F32); bias [N] of act_dtype or null;
 // y [M, N or N / 2] fp32 (out_f32) or act_dtype, row stride ldy.  gated: the N weight rows are groups of 64 = 32 gate rows followed by
 // the 32 up rows of the same channels (N % 64 == 0); y[m, c] = act(gate_c) * up_c.  act: 0 none, 1 relu, 2 silu, 3 gelu (tanh form), 4 tanh (on the gate,
-// or on the plain output).  softcap > 0: y <- softcap * tanh(y / softcap).
+// or on the plain output), 6 the square of relu.  softcap > 0: y <- softcap * tanh(y / softcap).
 extern "C" int mi355_dense_linear(const void* x, int32_t ldx, int32_t M, const void* w, int32_t N, int32_t K, const void* bias,
                                   void* y, int32_t ldy, int32_t out_f32, int32_t gated, int32_t act, float softcap,
                                   int32_t act_dtype, mi355_stream_t stream) {
@@ -490,7 +492,7 @@ extern "C" int mi355_dense_linear_ex(const void* x, int32_t ldx, int32_t M, cons
     MI355_CHECK_ARG(x && w && y && M > 0 && N > 0 && K > 0 && ldx >= K, "dense_linear: M=%d N=%d K=%d ldx=%d", M, N, K, ldx);
     MI355_CHECK_ARG(act_dtype == MI355_ACT_BF16 || act_dtype == MI355_ACT_F32, "dense_linear: act_dtype=%d (bf16 or fp32)", act_dtype);
     MI355_CHECK_ARG(!gated || N % 64 == 0, "dense_linear: gated needs N %% 64 == 0 (N=%d)", N);
-    MI355_CHECK_ARG(act >= 0 && act <= 5 && (act != DN_ACT_SWIGLU_CLAMP || (gated && act_param > 0.f)), "dense_linear: act=%d (gated=%d, parameter %g)", act, gated, (double)act_param);
+    MI355_CHECK_ARG(act >= 0 && act <= DN_ACT_RELU2 && (act != DN_ACT_SWIGLU_CLAMP || (gated && act_param > 0.f)), "dense_linear: act=%d (gated=%d, parameter %g)", act, gated, (double)act_param);
     MI355_CHECK_ARG(ldy >= (gated ? N / 2 : N), "dense_linear: ldy=%d", ldy);
     const bool bf = act_dtype == MI355_ACT_BF16;
     const size_t es = bf ? 2 : 4;
@@ -527,7 +529,7 @@ extern "C" int mi355_dense_linear_ex(const void* x, int32_t ldx, int32_t M, cons
     return MI355_OK;
 }
 
-// The same product for G groups in one launch (tile kernels at every M): group g uses the weight w + g * N * K ([G, N, K] contiguous) and
+// The same product for G groups in one launch: group g uses the weight w + g * N * K ([G, N, K] contiguous) and
 // bias + g * N, reads x from column xs * g on and writes y from column ys * g on.  offs null: every group takes all M rows (per-head
 // projections: xs, ys = the head's column step).  offs [G + 1] (device): M rows are sorted by group, group g owns rows offs[g] .. offs[g + 1] - 1;
 // sorted row r reads x row gather[r] (device, or null for r itself) and writes y row r (experts of a mixture: xs = ys = 0).  A row's result
@@ -551,7 +553,7 @@ extern "C" int mi355_dense_grouped_ex(const void* x, int32_t ldx, int32_t M, con
     MI355_CHECK_ARG(ldx >= xs * (G - 1) + K, "dense_grouped: ldx=%d for %d groups of K=%d at step %lld", ldx, G, K, (long long)xs);
     MI355_CHECK_ARG(act_dtype == MI355_ACT_BF16 || act_dtype == MI355_ACT_F32, "dense_grouped: act_dtype=%d (bf16 or fp32)", act_dtype);
     MI355_CHECK_ARG(!gated || N % 64 == 0, "dense_grouped: gated needs N %% 64 == 0 (N=%d)", N);
-    MI355_CHECK_ARG(act >= 0 && act <= 5 && (act != DN_ACT_SWIGLU_CLAMP || (gated && act_param > 0.f)), "dense_grouped: act=%d (gated=%d, parameter %g)", act, gated, (double)act_param);
+    MI355_CHECK_ARG(act >= 0 && act <= DN_ACT_RELU2 && (act != DN_ACT_SWIGLU_CLAMP || (gated && act_param > 0.f)), "dense_grouped: act=%d (gated=%d, parameter %g)", act, gated, (double)act_param);
     MI355_CHECK_ARG(ldy >= ys * (G - 1) + (gated ? N / 2 : N), "dense_grouped: ldy=%d", ldy);
     MI355_CHECK_ARG(G <= 65535 && (!gather || offs) && (!tiles || (offs && max_tiles > 0)), "dense_grouped: G=%d, gather and tiles need offs", G);
     const bool bf = act_dtype == MI355_ACT_BF16;
@@ -573,6 +575,20 @@ extern "C" int mi355_dense_grouped_ex(const void* x, int32_t ldx, int32_t M, con
         else    { if (gated) hipLaunchKernelGGL((dense_rows_grouped_kernel<float, 1, true>), grid, dim3(256), 0, st, p);
                   else       hipLaunchKernelGGL((dense_rows_grouped_kernel<float, 2, false>), grid, dim3(256), 0, st, p); }
         MI355_CHECK_LAUNCH("dense_rows_grouped_kernel");
+        return MI355_OK;
+    }
+    if (!offs && M <= 16) {                    // a decode step's rows through every group: the kernels of the plain linear, groups in the grid
+        const int nout = gated ? N / 2 : N, nt = (nout + 15) / 16;
+        if (bf && M > 1 && p.vec) {
+            const int nw = (nt * G >= 1024 || K < 1024) ? 4 : 8;
+            if (gated) hipLaunchKernelGGL(dense_skinny_bf16_kernel<true>, dim3(nt, G), dim3(64 * nw), 0, st, p, 0);
+            else       hipLaunchKernelGGL(dense_skinny_bf16_kernel<false>, dim3(nt, G), dim3(64 * nw), 0, st, p, 0);
+            MI355_CHECK_LAUNCH("dense_skinny_bf16_kernel");
+            return MI355_OK;
+        }
+        if (bf) { if (gated) launch_rows<bf16, true>(p, st); else launch_rows<bf16, false>(p, st); }
+        else    { if (gated) launch_rows<float, true>(p, st); else launch_rows<float, false>(p, st); }
+        MI355_CHECK_LAUNCH("dense_rows_kernel");
         return MI355_OK;
     }
     if (bf) {

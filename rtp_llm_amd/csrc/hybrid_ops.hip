@@ -281,6 +281,146 @@ __global__ __launch_bounds__(256) void hy_branch_norm_kernel(float* x, BranchTer
     }
 }
 
+// ------------------------------------------------------------------------------------------------ parallel residual streams: write back, read, norm
+// The residual is S streams X[r, s] (fp32 [rows, S, W]).  One launch ends a sublayer and starts the next:
+//     X_t <- sum_s mix[s, t] X_s + wr[t] y      (all new streams from the old ones),
+//     h   <- N(sum_t rd[t] X_t) * w             (RMS norm under the next sublayer's weight; rd null: the plain sum of the streams)
+// with the ended sublayer's result y = ca A + cb B (+ a mixture's weighted sum), A and B RMS-normed over the row under na / nb first when those are given.
+// ids non-null (the start of the model): every stream is the token's embedding row instead.  rows non-null: only these rows are formed and the
+// streams are not written (the last norm, on the rows whose logits are asked for).  h null: the streams are only written.
+struct StreamTerms { const float* a; float ca; const void* na; const float* b; float cb; const void* nb; float neps; };
+struct StreamMix { const float* mix; const float* wr; const float* rd; int S; };
+
+template <typename T, bool VEC, int SM>
+__global__ __launch_bounds__(256) void hy_streams_kernel(float* X, StreamTerms st, MoeSum ms, StreamMix sm, const int32_t* ids, const T* table, int vocab,
+                                                         const int32_t* rows, const T* w, float eps, int W, T* h) {
+    extern __shared__ __attribute__((aligned(16))) float hy_xs[];
+    __shared__ float red[4];
+    constexpr int V = VEC ? 4 : 1, KMAX = 8;
+    const int r = blockIdx.x, src = rows ? rows[r] : r, S = sm.S;
+    const size_t base = (size_t)src * W;
+    float* xr = X + (size_t)src * S * W;
+    const T* emb = nullptr;
+    if (ids) { int id = ids[src]; id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id); emb = table + (size_t)id * W; }
+    float ca = st.ca, cb = st.cb;
+    if (st.na || st.nb) {                                    // the branches' own norms
+        float sa = 0.f, sb = 0.f;
+        for (int c = threadIdx.x * V; c < W; c += 256 * V) {
+            float t[4] = {0.f, 0.f, 0.f, 0.f};
+            if (st.na) {
+                if (VEC) hy_load4<float>(st.a + base + c, t); else t[0] = st.a[base + c];
+#pragma unroll
+                for (int e = 0; e < V; ++e) sa = __builtin_fmaf(t[e], t[e], sa);
+            }
+            if (st.nb) {
+                if (VEC) hy_load4<float>(st.b + base + c, t); else t[0] = st.b[base + c];
+#pragma unroll
+                for (int e = 0; e < V; ++e) sb = __builtin_fmaf(t[e], t[e], sb);
+            }
+        }
+        __shared__ float red2[4];
+        sa = hy_wave_sum(sa); sb = hy_wave_sum(sb);
+        if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sa; red2[threadIdx.x >> 6] = sb; }
+        __syncthreads();
+        if (st.na) ca *= 1.f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)W + st.neps);
+        if (st.nb) cb *= 1.f / sqrtf(((red2[0] + red2[1]) + (red2[2] + red2[3])) / (float)W + st.neps);
+        __syncthreads();
+    }
+    float mw[KMAX];
+    const float* my[KMAX];
+    if (ms.y) {
+#pragma unroll
+        for (int k = 0; k < KMAX; ++k)
+            if (k < ms.top) { mw[k] = ms.wts[(size_t)src * ms.top + k]; my[k] = ms.y + (size_t)ms.place[(size_t)src * ms.top + k] * W; }
+    }
+    float ss = 0.f;
+    for (int c = threadIdx.x * V; c < W; c += 256 * V) {
+        float v[SM][4], u[4] = {0.f, 0.f, 0.f, 0.f}, t[4] = {0.f, 0.f, 0.f, 0.f};
+        if (emb) {
+            if (VEC) hy_load4<T>(emb + c, t); else t[0] = (float)emb[c];
+#pragma unroll
+            for (int s = 0; s < SM; ++s)
+                if (s < S) {
+                    if (!rows) { if (VEC) hy_store4<float>(xr + (size_t)s * W + c, t); else xr[(size_t)s * W + c] = t[0]; }
+                    const float f = sm.rd ? sm.rd[s] : 1.f;
+#pragma unroll
+                    for (int e = 0; e < V; ++e) u[e] = __builtin_fmaf(f, t[e], u[e]);
+                }
+        } else {
+#pragma unroll
+            for (int s = 0; s < SM; ++s)
+                if (s < S) { if (VEC) hy_load4<float>(xr + (size_t)s * W + c, v[s]); else v[s][0] = xr[(size_t)s * W + c]; }
+            float y[4] = {0.f, 0.f, 0.f, 0.f}, g[4];
+            if (st.a) {
+                if (VEC) hy_load4<float>(st.a + base + c, t); else t[0] = st.a[base + c];
+                if (st.na) { if (VEC) hy_load4<T>((const T*)st.na + c, g); else g[0] = (float)((const T*)st.na)[c]; }
+#pragma unroll
+                for (int e = 0; e < V; ++e) y[e] = ca * t[e] * (st.na ? g[e] : 1.f);
+            }
+            if (st.b) {
+                if (VEC) hy_load4<float>(st.b + base + c, t); else t[0] = st.b[base + c];
+                if (st.nb) { if (VEC) hy_load4<T>((const T*)st.nb + c, g); else g[0] = (float)((const T*)st.nb)[c]; }
+#pragma unroll
+                for (int e = 0; e < V; ++e) y[e] += cb * t[e] * (st.nb ? g[e] : 1.f);
+            }
+            if (ms.y) {                                      // the chosen experts in choice order
+                float sum[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int k = 0; k < KMAX; ++k) {
+                    if (k >= ms.top) break;
+                    if (VEC) hy_load4<float>(my[k] + c, t); else t[0] = my[k][c];
+#pragma unroll
+                    for (int e = 0; e < V; ++e) sum[e] = __builtin_fmaf(mw[k], t[e], sum[e]);
+                }
+                for (int k = KMAX; k < ms.top; ++k) {
+                    const float wk = ms.wts[(size_t)src * ms.top + k];
+                    const float* yr = ms.y + (size_t)ms.place[(size_t)src * ms.top + k] * W + c;
+                    if (VEC) hy_load4<float>(yr, t); else t[0] = yr[0];
+#pragma unroll
+                    for (int e = 0; e < V; ++e) sum[e] = __builtin_fmaf(wk, t[e], sum[e]);
+                }
+#pragma unroll
+                for (int e = 0; e < V; ++e) y[e] += sum[e];
+            }
+#pragma unroll
+            for (int to = 0; to < SM; ++to)
+                if (to < S) {
+                    float nv[4] = {0.f, 0.f, 0.f, 0.f};
+                    if (sm.mix) {
+                        const float o = sm.wr[to];
+#pragma unroll
+                        for (int e = 0; e < V; ++e) nv[e] = o * y[e];
+#pragma unroll
+                        for (int s = 0; s < SM; ++s)
+                            if (s < S) {
+                                const float f = sm.mix[s * S + to];
+#pragma unroll
+                                for (int e = 0; e < V; ++e) nv[e] = __builtin_fmaf(f, v[s][e], nv[e]);
+                            }
+                        if (!rows) { if (VEC) hy_store4<float>(xr + (size_t)to * W + c, nv); else xr[(size_t)to * W + c] = nv[0]; }
+                    } else {
+#pragma unroll
+                        for (int e = 0; e < V; ++e) nv[e] = v[to][e];
+                    }
+                    const float f = sm.rd ? sm.rd[to] : 1.f;
+#pragma unroll
+                    for (int e = 0; e < V; ++e) u[e] = __builtin_fmaf(f, nv[e], u[e]);
+                }
+        }
+#pragma unroll
+        for (int e = 0; e < V; ++e) { hy_xs[c + e] = u[e]; ss = __builtin_fmaf(u[e], u[e], ss); }
+    }
+    if (!h) return;
+    const float inv = 1.f / sqrtf(hy_block_sum(ss, red) / (float)W + eps);
+    for (int c = threadIdx.x * V; c < W; c += 256 * V) {
+        float g[4], o[4];
+        if (VEC) hy_load4<T>(w + c, g); else g[0] = (float)w[c];
+#pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = hy_xs[c + e] * inv * g[e];
+        if (VEC) hy_store4<T>(h + (size_t)r * W + c, o); else h[(size_t)r * W + c] = (T)o[0];
+    }
+}
+
 // ------------------------------------------------------------------------------------------------ residual update + weighted average over depth + norm
 // A layer's own result X_n = x + a (a: the layer's last branch, may be null) joins the per-step stack of earlier results (stack[j] = X_j, planes
 // of `plane` floats; X_0 is the embedding output), and what the next layer reads is x <- sum_{j <= n} coef[j] X_j, summed in the order j = 0 .. n in
@@ -457,7 +597,11 @@ __device__ __forceinline__ float hy_lane_f(float v, int j) { return __builtin_bi
 // Optional parts of the mask, the scores and the output (AttnExtra): window > 0: a row at position i sees keys j with 0 <= i - j < window;
 // softcap > 0: score <- softcap tanh(score / softcap) after the scale; ogate non-null: head h of row r is multiplied by
 // sigmoid(ogate[r * ldg + h]) (fp32 pre-activations, one number per head).
-struct AttnExtra { int window; float softcap; const float* ogate; int ldg; };
+// (gate_channels: one number per value channel instead, ogate[r * ldg + h * vdim + c]).
+struct AttnExtra { int window; float softcap; const float* ogate; int ldg; int gate_channels; };
+__device__ __forceinline__ float hy_channel_gate(const AttnExtra& ex, int r, int h, int vdim, int c) {
+    return ex.gate_channels ? hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h * vdim + c]) : 1.f;
+}
 __device__ __forceinline__ int hy_first_visible(int p, int chunk, int window) {
     return chunk > 0 ? (p / chunk) * chunk : (window > 0 ? max(0, p - window + 1) : 0);
 }
@@ -610,7 +754,7 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
     float lt = 0.f;
     for (int w = 0; w < NW; ++w) lt = __builtin_fmaf(l_s[w], (m_s[w] == -INFINITY) ? 0.f : expf(m_s[w] - mm), lt);
     float invl = S > 1 ? 1.f : (lt > 0.f ? 1.f / lt : 0.f);
-    if (S == 1 && ex.ogate) invl *= hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h]);
+    if (S == 1 && ex.ogate && !ex.gate_channels) invl *= hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h]);
     for (int c = tid; c < g.vdim; c += NT) {
         float a = 0.f;
         for (int w = 0; w < NW; ++w) a = __builtin_fmaf(acc_s[w][c], (m_s[w] == -INFINITY) ? 0.f : expf(m_s[w] - mm), a);
@@ -632,10 +776,10 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
             float sn, cs;
             sincosf(fp * vfreq[mi], &sn, &cs);
             const float a = o_s[c0], b = o_s[c1];
-            od[c0] = (T)(a * cs + b * sn); od[c1] = (T)(b * cs - a * sn);
+            od[c0] = (T)((a * cs + b * sn) * hy_channel_gate(ex, r, h, g.vdim, c0)); od[c1] = (T)((b * cs - a * sn) * hy_channel_gate(ex, r, h, g.vdim, c1));
         }
     } else {
-        for (int c = tid; c < g.vdim; c += NT) od[c] = (T)o_s[c];
+        for (int c = tid; c < g.vdim; c += NT) od[c] = (T)(o_s[c] * hy_channel_gate(ex, r, h, g.vdim, c));
     }
 }
 
@@ -653,7 +797,7 @@ __global__ __launch_bounds__(256) void hy_attn_merge_kernel(const float* parts, 
         lt = __builtin_fmaf(pd[(size_t)s_ * (g.vdim + 2) + 1], (ms == -INFINITY) ? 0.f : expf(ms - mm), lt);
     }
     float invl = lt > 0.f ? 1.f / lt : 0.f;
-    if (ex.ogate) invl *= hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h]);
+    if (ex.ogate && !ex.gate_channels) invl *= hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h]);
     for (int c = tid; c < g.vdim; c += 256) {
         float a = 0.f;
         for (int s_ = 0; s_ < S; ++s_) {
@@ -672,10 +816,10 @@ __global__ __launch_bounds__(256) void hy_attn_merge_kernel(const float* parts, 
             float sn, cs;
             sincosf(fp * vfreq[mi], &sn, &cs);
             const float a = o_s[c0], b = o_s[c1];
-            od[c0] = (T)(a * cs + b * sn); od[c1] = (T)(b * cs - a * sn);
+            od[c0] = (T)((a * cs + b * sn) * hy_channel_gate(ex, r, h, g.vdim, c0)); od[c1] = (T)((b * cs - a * sn) * hy_channel_gate(ex, r, h, g.vdim, c1));
         }
     } else {
-        for (int c = tid; c < g.vdim; c += 256) od[c] = (T)o_s[c];
+        for (int c = tid; c < g.vdim; c += 256) od[c] = (T)(o_s[c] * hy_channel_gate(ex, r, h, g.vdim, c));
     }
 }
 
@@ -859,7 +1003,7 @@ __global__ __launch_bounds__(256) void hy_attn_tiles_kernel(const float* q, int 
         const int row = lq * 4 + e;
         const float lt = hy_sum16(l[e]);
         float inv = lt > 0.f ? 1.f / lt : 0.f;
-        if (ex.ogate && row < n) inv *= hy_sigmoid(ex.ogate[(size_t)(r0 + row) * ex.ldg + h]);
+        if (ex.ogate && !ex.gate_channels && row < n) inv *= hy_sigmoid(ex.ogate[(size_t)(r0 + row) * ex.ldg + h]);
         const float fp = (float)(p0 + row);
         bf16* od = out + ((size_t)(r0 + row) * g.H + h) * g.vdim;
 #pragma unroll
@@ -883,7 +1027,7 @@ __global__ __launch_bounds__(256) void hy_attn_tiles_kernel(const float* q, int 
                 sincosf(fp * vfreq[mi], &sn, &cs);
                 v = first ? (v * cs + other * sn) : (v * cs - other * sn);
             }
-            if (row < n) od[c] = (bf16)v;
+            if (row < n) od[c] = (bf16)(v * hy_channel_gate(ex, r0 + row, h, g.vdim, c));
         }
     }
     }   // pass
@@ -920,17 +1064,17 @@ __global__ __launch_bounds__(256) void hy_chunk_plan_kernel(const int32_t* row_s
 }
 
 __global__ __launch_bounds__(256) void hy_chunk_prefix_kernel(const int32_t* cs, const int32_t* sc, const int32_t* slot, const int32_t* first_pos, const float* decay,
-                                                              int H, int per_head, float* chunk_state, float* state) {
+                                                              int H, int per_head, float* chunk_state, float* state, const float* cdecay) {
     const int sq = blockIdx.x, h = blockIdx.y, e = blockIdx.z * 256 + threadIdx.x;
     if (e >= per_head) return;
-    const float a = decay[h];
+    const float a = cdecay ? 0.f : decay[h];              // cdecay [chunks, H]: every chunk's own total decay
     float* st = state + ((size_t)slot[sq] * H + h) * per_head + e;
     float S = first_pos[sq] == 0 ? 0.f : *st;
     for (int c = sc[sq]; c < sc[sq + 1]; ++c) {
         float* cp = chunk_state + ((size_t)c * H + h) * per_head + e;
         const float L = *cp;
         *cp = S;
-        S = __builtin_fmaf(hy_decay_pow(a, cs[c + 1] - cs[c]), S, L);
+        S = __builtin_fmaf(cdecay ? cdecay[(size_t)c * H + h] : hy_decay_pow(a, cs[c + 1] - cs[c]), S, L);
     }
     *st = S;
 }
@@ -941,6 +1085,72 @@ __global__ __launch_bounds__(256) void hy_chunk_prefix_kernel(const int32_t* cs,
 // decay, rank-one update, partial q . S), and the DS partial outputs per token are summed from LDS.  Short RD keeps the dependent chain per
 // token short; the walk itself is the sequential part of the recurrence.
 enum { SCAN_HGRN2 = 0, SCAN_GLA = 1, SCAN_FIXED = 2, SCAN_FIXED_SILU = 3 };
+
+// Matrix memory under exponential gates (MEM instances of the scan kernel).  Per head log gates i (input) and f (forget) and a running maximum m that keeps
+// the exponentials in range:  m_t = max(f_t + m_(t-1), i_t),  keep_t = e^(f_t + m_(t-1) - m_t),  take_t = e^(i_t - m_t),
+//     S_t = keep_t S_(t-1) + take_t k_t v_t^T,   n_t = keep_t n_(t-1) + take_t k_t,   o_t = S_t^T q_t / (max(|n_t . q_t|, e^(-m_t)) + den_eps).
+// m is a maximum over (running sum of f) + i, an associative scan: a wave forms it for the tokens of a pass from lane shuffles.  The kernel leaves
+// S_t^T q_t and the denominators (one per row and head); the norm that follows divides.  A head's state is [dim * vdim | dim]: S, then n.
+struct MemGates {
+    int io, fo;                  // columns of the gates' pre-activations (H each, biases included) in proj
+    float cap;                   // both pre-activations pass cap tanh(z / cap); the forget gate is the log sigmoid of that
+    float den_eps;
+    const float* gates;          // null: formed here; else fp32 [rows, H, 3] = keep, take, e^(-m) (hy_memory_gates_kernel)
+    float* mstate; int nz;       // running maximum [slots, H, nz]: every value-column block of the grid has a copy of its own
+    float* cdecay;               // null, or fp32 [sequences, H]: receives the product of the sequence's keeps
+    float* den;                  // fp32 [rows, H]
+    int raw;                     // den receives n . q itself (a later read-only pass completes it)
+};
+
+__device__ __forceinline__ float hy_log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+
+// Inclusive scan over the first `width` lanes (a power of two) of the pairs (F, M): (F1, M1) then (F2, M2) is (F1 + F2, max(M1 + F2, M2)).
+__device__ __forceinline__ void hy_maxplus_scan(float& F, float& M, int lane, int width) {
+    for (int o = 1; o < width; o <<= 1) {
+        const float F1 = __shfl_up(F, o, 64), M1 = __shfl_up(M, o, 64);
+        if (lane >= o) { M = fmaxf(M1 + F, M); F = F1 + F; }
+    }
+}
+
+// The gates of every token of every sequence for the chunked form: one block per (sequence, head), 1024 tokens a trip.
+__global__ __launch_bounds__(1024) void hy_memory_gates_kernel(const float* proj, int ld, MemGates g, int H, const int32_t* row_start, const int32_t* slot,
+                                                               const int32_t* first_pos, float* out) {
+    __shared__ float wF[16], wM[16], mlast[16];
+    const int sq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int r0 = row_start[sq], r1 = row_start[sq + 1];
+    float* ms = g.mstate + ((size_t)slot[sq] * H + h) * g.nz;
+    float m_run = first_pos[sq] == 0 ? 0.f : ms[0];
+    for (int t0 = r0; t0 < r1; t0 += 1024) {
+        const int t = t0 + tid, last = min(1024, r1 - t0) - 1;
+        float li = -INFINITY, lf = 0.f;
+        if (t < r1) {
+            const float* row = proj + (size_t)t * ld;
+            li = g.cap * tanhf(row[g.io + h] / g.cap);
+            lf = hy_log_sigmoid(g.cap * tanhf(row[g.fo + h] / g.cap));
+        }
+        float F = lf, M = li;
+        hy_maxplus_scan(F, M, lane, 64);
+        if (lane == 63) { wF[wave] = F; wM[wave] = M; }
+        __syncthreads();
+        float Fp = 0.f, Mp = -INFINITY;                     // the waves before this one
+        for (int w = 0; w < wave; ++w) { Mp = fmaxf(Mp + wF[w], wM[w]); Fp += wF[w]; }
+        const float m = fmaxf(fmaxf(m_run + Fp, Mp) + F, M);
+        if (lane == 63) mlast[wave] = m;
+        __syncthreads();
+        float prev = __shfl_up(m, 1, 64);
+        if (lane == 0) prev = wave == 0 ? m_run : mlast[wave - 1];
+        if (t < r1) {
+            float* o = out + ((size_t)t * H + h) * 3;
+            o[0] = expf(lf + prev - m); o[1] = expf(li - m); o[2] = expf(-m);
+        }
+        // the running maximum after the trip's last token
+        if (tid == last) wF[0] = m;
+        __syncthreads();
+        m_run = wF[0];
+        __syncthreads();
+    }
+    if (tid < g.nz) ms[tid] = m_run;
+}
 
 struct ScanParams {
     const float* proj; int ld; int qo, ko, vo;     // fp32 projections [rows, ld]: q, k (GLA) or forget pre-activation (HGRN2), v at these columns
@@ -953,24 +1163,34 @@ struct ScanParams {
     float* out;                                     // [rows, H * vdim]
     int tok;                                        // tokens staged per pass
     int apply;                                      // fixed-decay modes: the state is only read: out[t] += decay^(t - first row + 1) * (S^T q_t), nothing is written back
+    MemGates mem;                                   // MEM instances (apply: out[t] += (product of the keeps up to t) * (S^T q_t), den completed likewise)
 };
 
-template <typename T, int RD>
+template <typename T, int RD, bool MEM = false>
 __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
     extern __shared__ __attribute__((aligned(16))) float hy_sm[];
     const int DS = blockDim.x >> 6, dpad = DS * RD, TOK = p.tok;
     float* q_s = hy_sm;                          // [TOK][dpad]
     float* k_s = q_s + TOK * dpad;
-    float* a_s = k_s + TOK * dpad;
+    float* a_s = k_s + TOK * dpad;               // MEM: the products n . q, one per key row, summed after the walk
     float* v_s = a_s + TOK * dpad;               // [TOK][64]
     float* part_s = v_s + TOK * 64;              // [TOK][DS][64]
     const int sq = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * 64;
     const int tid = threadIdx.x, c = tid & 63, ds = tid >> 6;
     const int r0 = p.row_start[sq], r1 = p.row_start[sq + 1];
     const bool vok = v0 + c < p.vdim;
-    float* st = p.state + (((size_t)p.slot[sq] * p.H + h) * p.dim) * p.vdim + v0 + c;
+    float* sth = p.state + ((size_t)p.slot[sq] * p.H + h) * p.dim * (MEM ? p.vdim + 1 : p.vdim);
+    float* st = sth + v0 + c;
     float s[RD];
     const bool fresh = p.first_pos[sq] == 0;
+    // MEM: the block of the first value columns also carries n, row d = ds * RD + c of it in lane c < RD of wave ds
+    __shared__ float keep_s[16], take_s[16], em_s[16];
+    const bool own_n = MEM && v0 == 0 && c < RD;
+    float n = 0.f, P = 1.f, m_run = 0.f, ri = 0.f, rf = 0.f, re = 0.f;
+    if constexpr (MEM) {
+        if (own_n && !fresh && ds * RD + c < p.dim) n = sth[(size_t)p.dim * p.vdim + ds * RD + c];
+        if (!fresh && !p.mem.gates) m_run = p.mem.mstate[((size_t)p.slot[sq] * p.H + h) * p.mem.nz + blockIdx.z];
+    }
 #pragma unroll
     for (int j = 0; j < RD; ++j) {
         const int d = ds * RD + j;
@@ -1000,10 +1220,35 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             rv[e] = 0.f;
             if (i < nt * 64 && v0 + (i & 63) < p.vdim) rv[e] = p.proj[(size_t)(t0 + (i >> 6)) * p.ld + p.vo + h * p.vdim + v0 + (i & 63)];
         }
+        if constexpr (MEM) {
+            if (tid < nt) {
+                const size_t t = t0 + tid;
+                if (p.mem.gates) { const float* gp = p.mem.gates + (t * p.H + h) * 3; ri = gp[0]; rf = gp[1]; re = gp[2]; }
+                else { ri = p.proj[t * p.ld + p.mem.io + h]; rf = p.proj[t * p.ld + p.mem.fo + h]; }
+            }
+        }
     };
     if (r0 < r1) fetch(r0);
     for (int t0 = r0; t0 < r1; t0 += TOK) {
         const int nt = min(TOK, r1 - t0);
+        if constexpr (MEM) {
+            if (tid < 64) {
+                float keep = ri, take = rf, em = re;
+                if (!p.mem.gates) {
+                    const float li = tid < nt ? p.mem.cap * tanhf(ri / p.mem.cap) : -INFINITY;
+                    const float lf = tid < nt ? hy_log_sigmoid(p.mem.cap * tanhf(rf / p.mem.cap)) : 0.f;
+                    float F = lf, M = li;
+                    hy_maxplus_scan(F, M, tid, 16);
+                    const float m = fmaxf(m_run + F, M);
+                    float prev = __shfl_up(m, 1, 64);
+                    if (tid == 0) prev = m_run;
+                    keep = expf(lf + prev - m); take = expf(li - m); em = expf(-m);
+                    m_run = __shfl(m, nt - 1, 64);
+                }
+                if (tid < nt) { keep_s[tid] = keep; take_s[tid] = take; em_s[tid] = em; }
+            }
+            __syncthreads();
+        }
 #pragma unroll
         for (int e = 0; e < EL; ++e) {
             const int i = tid + e * blockDim.x, d = i % dpad;
@@ -1011,7 +1256,9 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             float qv = 0.f, kv = 0.f, av = 1.f;
             if (d < p.dim) {
                 const int hd = h * p.dim + d;
-                if (p.mode == SCAN_FIXED) {          // one decay per head (fp32 [H] behind `lower`), q and k as given
+                if constexpr (MEM) {
+                    qv = rq[e] * p.qscale; kv = rk[e] * take_s[i / dpad];
+                } else if (p.mode == SCAN_FIXED) {          // one decay per head (fp32 [H] behind `lower`), q and k as given
                     qv = rq[e]; kv = rk[e]; av = ((const float*)p.lower)[h];
                 } else if (p.mode == SCAN_FIXED_SILU) {   // the same decay; q, k (and v below) pass through silu first
                     qv = hy_silu(rq[e]); kv = hy_silu(rk[e]); av = ((const float*)p.lower)[h];
@@ -1025,7 +1272,8 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
                     qv = rq[e] * p.qscale; kv = rk[e]; av = expf(ls / p.tau);
                 }
             }
-            q_s[i] = qv; k_s[i] = kv; a_s[i] = av;
+            q_s[i] = qv; k_s[i] = kv;
+            if constexpr (!MEM) a_s[i] = av;
         }
 #pragma unroll
         for (int e = 0; e < VE; ++e) {
@@ -1044,6 +1292,16 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             const f32x4* kk = (const f32x4*)(k_s + t * dpad + ds * RD);
             const f32x4* aa = (const f32x4*)(a_s + t * dpad + ds * RD);
             float o[4] = {0.f, 0.f, 0.f, 0.f};
+            float keep = 1.f;
+            if constexpr (MEM) {
+                keep = keep_s[t];
+                P *= keep;
+                if (own_n) {
+                    const int i = t * dpad + ds * RD + c;
+                    if (!p.apply) n = __builtin_fmaf(keep, n, k_s[i]);
+                    a_s[i] = n * q_s[i] * (p.apply ? P : 1.f);
+                }
+            }
             if (p.apply) {
 #pragma unroll
                 for (int j4 = 0; j4 < RD / 4; ++j4) {
@@ -1054,7 +1312,7 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             } else {
 #pragma unroll
                 for (int j4 = 0; j4 < RD / 4; ++j4) {
-                    const f32x4 a4 = aa[j4], k4 = kk[j4], q4 = qq[j4];
+                    const f32x4 a4 = MEM ? f32x4{keep, keep, keep, keep} : aa[j4], k4 = kk[j4], q4 = qq[j4];
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         const int j = j4 * 4 + e;
@@ -1063,7 +1321,7 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
                     }
                 }
             }
-            part_s[(t * DS + ds) * 64 + c] = (o[0] + o[1]) + (o[2] + o[3]);
+            part_s[(t * DS + ds) * 64 + c] = ((o[0] + o[1]) + (o[2] + o[3])) * (MEM && p.apply ? P : 1.f);
         }
         __syncthreads();
         for (int i = tid; i < nt * 64; i += blockDim.x) {
@@ -1072,8 +1330,21 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             float o = 0.f;
             for (int k = 0; k < DS; ++k) o += part_s[(t * DS + k) * 64 + cc];
             float* dst = p.out + (size_t)(t0 + t) * p.H * p.vdim + h * p.vdim + v0 + cc;
-            if (p.apply) *dst += o * hy_decay_pow(((const float*)p.lower)[h], t0 + t - r0 + 1);
+            if (p.apply) *dst += MEM ? o : o * hy_decay_pow(((const float*)p.lower)[h], t0 + t - r0 + 1);
             else *dst = o;
+        }
+        if constexpr (MEM) {
+            if (v0 == 0)
+                for (int t = ds; t < nt; t += DS) {          // a wave per token
+                    float nq = 0.f;
+                    for (int d = c; d < dpad; d += 64) nq += a_s[t * dpad + d];
+                    nq = hy_wave_sum(nq);
+                    float* dp = p.mem.den + (size_t)(t0 + t) * p.H + h;
+                    if (c == 0) {
+                        if (p.apply) nq += *dp;
+                        *dp = p.mem.raw ? nq : fmaxf(fabsf(nq), em_s[t]) + p.mem.den_eps;
+                    }
+                }
         }
     }
     if (vok && !p.apply) {
@@ -1083,6 +1354,85 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
             if (d < p.dim) st[(size_t)d * p.vdim] = s[j];
         }
     }
+    if constexpr (MEM) {
+        if (own_n && !p.apply && ds * RD + c < p.dim) sth[(size_t)p.dim * p.vdim + ds * RD + c] = n;
+        if (tid == 0) {
+            if (!p.mem.gates) p.mem.mstate[((size_t)p.slot[sq] * p.H + h) * p.mem.nz + blockIdx.z] = m_run;
+            if (p.mem.cdecay && v0 == 0) p.mem.cdecay[(size_t)sq * p.H + h] = P;
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ short causal convolutions in front of a recurrence
+// Channels [0, C) of the fp32 projection rows each pass a causal convolution over time (taps weights, the last one on the current token) and silu.
+// The first `units` heads of `dim` channels (query heads, then key heads) are then brought to unit length, x / sqrt(sum x^2 + unit_eps), the first
+// `uq` of them also multiplied by qscale.  Columns lo .. lo + R - 1 of the projections are rounded to the activation type in the same launch (inputs of
+// the low-rank products that follow).  Before a sequence's first row of the step stand the taps - 1 rows its slot keeps (fp32 [slots, taps - 1, C]; zeros
+// before position 0); the kernel that runs the recurrence afterwards moves the slot's rows on (hy_conv_advance): here they are only read.
+struct ConvParams {
+    const float* proj; int ld; int C, taps;
+    const void* w;                                  // [C, taps], activation type
+    int units, uq, dim; float qscale, unit_eps;
+    const float* hist;                              // [slots, taps - 1, C]
+    const int32_t* seq; const int32_t* row_start; const int32_t* slot; const int32_t* first_pos;
+    float* out;                                     // [rows, C]
+    int lo, R; void* low;                           // low [rows, R] of the activation type (null: none)
+};
+
+constexpr int CONV_PIECE = 256;                     // channels of a wave's piece outside the unit heads
+
+template <typename T>
+__global__ __launch_bounds__(256) void hy_short_conv_kernel(ConvParams p, int pieces_v, int pieces) {
+    const int r = blockIdx.x, lane = threadIdx.x & 63, piece = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (piece >= pieces) return;
+    if (piece >= p.units + pieces_v) {              // the low-rank inputs
+        const int b = (piece - p.units - pieces_v) * CONV_PIECE;
+        for (int c = b + lane; c < min(b + CONV_PIECE, p.R); c += 64) ((T*)p.low)[(size_t)r * p.R + c] = (T)p.proj[(size_t)r * p.ld + p.lo + c];
+        return;
+    }
+    const bool head = piece < p.units;
+    const int c0 = head ? piece * p.dim : p.units * p.dim + (piece - p.units) * CONV_PIECE;
+    const int c1 = head ? c0 + p.dim : min(c0 + CONV_PIECE, p.C);
+    const int sq = p.seq[r], i = r - p.row_start[sq], pos = p.first_pos[sq] + i, K = p.taps - 1;
+    const float* hist = p.hist + (size_t)p.slot[sq] * K * p.C;
+    constexpr int NC = 8;                           // channels per lane kept in registers (unit heads of up to 512 channels)
+    float v[NC], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < NC; ++e) {
+        const int c = c0 + lane + 64 * e;
+        v[e] = 0.f;
+        if (c >= c1) continue;
+        float a = 0.f;
+        for (int j = 0; j < p.taps; ++j) {
+            const int back = K - j;                 // tokens before this one
+            float x = 0.f;
+            if (back <= i) x = p.proj[(size_t)(r - back) * p.ld + c];
+            else if (back <= pos) x = hist[(size_t)(K + i - back) * p.C + c];
+            a = __builtin_fmaf((float)((const T*)p.w)[(size_t)c * p.taps + j], x, a);
+        }
+        v[e] = hy_silu(a);
+        ss = __builtin_fmaf(v[e], v[e], ss);
+    }
+    float f = 1.f;
+    if (head) f = 1.f / sqrtf(hy_wave_sum(ss) + p.unit_eps) * (piece < p.uq ? p.qscale : 1.f);
+#pragma unroll
+    for (int e = 0; e < NC; ++e) {
+        const int c = c0 + lane + 64 * e;
+        if (c < c1) p.out[(size_t)r * p.C + c] = v[e] * f;
+    }
+}
+
+// The slot's last taps - 1 raw rows after the step, channels c = first, first + step, ...: rows of this step, or older ones moved up.
+__device__ __forceinline__ void hy_conv_advance(const float* raw, int ld, int C, int taps, float* hist, int r0, int r1, int first_pos, int first, int step) {
+    const int K = taps - 1, n = r1 - r0;
+    for (int c = first; c < C; c += step)
+        for (int j = 0; j < K; ++j) {               // row j stands for the token K - j before the next one
+            const int back = K - j;
+            float x = 0.f;
+            if (back <= n) x = raw[(size_t)(r1 - back) * ld + c];
+            else if (back <= first_pos + n) x = hist[(size_t)(j + n) * C + c];
+            hist[(size_t)j * C + c] = x;
+        }
 }
 
 // ------------------------------------------------------------------------------------------------ generalized delta rule
@@ -1099,7 +1449,14 @@ struct DeltaParams {
     const int32_t* row_start; const int32_t* slot; const int32_t* first_pos;
     float* state;                                     // [slots, H, dim, vdim]
     float* out;                                       // [rows, H * vdim]
+    // CHANNEL instances: S <- g * S (a decay per key channel), u = beta (v - S^T k), S <- S + k u^T, o = S^T r.  r and k: G heads (head h reads h / (H / G)) as
+    // given; g = exp(-rate[h] softplus(z + zbias)), beta = sigmoid of one pre-activation per head (bp [rows, ldb]).  Over the old state that is
+    // S_new = diag(g) S + (beta k)(v - (g k)^T S)^T.  hist non-null: the short convolution's rows of the slot are moved on (raw, ldr, C, taps).
+    int G; const float* zbias; const float* rate; const float* bp; int ldb;
+    const float* raw; int ldr, C, taps; float* hist;
 };
+
+__device__ __forceinline__ float hy_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
 template <int LPC> __device__ __forceinline__ float hy_lanes_sum(float v);
 template <> __device__ __forceinline__ float hy_lanes_sum<4>(float v) {
@@ -1111,7 +1468,7 @@ template <> __device__ __forceinline__ float hy_lanes_sum<16>(float v) { return 
 // LPC lanes (4 or 16, neighbours inside a DPP row) own one value column, each RD key rows of it (dim <= LPC * RD); a wave owns 64 / LPC columns and a
 // block of four waves CW = 256 / LPC.  Sixteen lanes per column keep the per-token chain short (RD multiply-adds, four DPP steps), which is what a
 // single sequence's walk is bound by; TOK tokens are staged per pass, and the raw projections of the next pass are fetched during the walk.
-template <int RD, int LPC>
+template <int RD, int LPC, bool CHANNEL = false>
 __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
     constexpr int dpad = LPC * RD, CW = 256 / LPC, TOK = dpad <= 128 ? 16 : 8;
     constexpr int EL = (TOK * dpad + 255) / 256, VE = (TOK * CW + 255) / 256;
@@ -1130,6 +1487,7 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
         S[j] = (!fresh && vok && d < p.dim) ? st[(size_t)d * p.vdim] : 0.f;
     }
     float fr[EL], fk[EL], fa[EL], fz[EL], fv[VE];
+    const int kvh = CHANNEL ? h / (p.H / p.G) : h;
     auto fetch = [&](int t0) {
         const int nt = min(TOK, r1 - t0);
 #pragma unroll
@@ -1139,8 +1497,13 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             if (i < nt * dpad && d < p.dim) {
                 const float* row = p.proj + (size_t)(t0 + t) * p.ld;
                 const int hd = h * p.dim + d;
-                fr[e] = row[p.ro + hd]; fk[e] = row[p.ko + hd]; fa[e] = row[p.ao + hd];
-                fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd];
+                if constexpr (CHANNEL) {
+                    fr[e] = row[p.ro + kvh * p.dim + d]; fk[e] = row[p.ko + kvh * p.dim + d]; fa[e] = p.bp[(size_t)(t0 + t) * p.ldb + h];
+                    fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd] + p.zbias[hd];
+                } else {
+                    fr[e] = row[p.ro + hd]; fk[e] = row[p.ko + hd]; fa[e] = row[p.ao + hd];
+                    fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd];
+                }
             }
         }
 #pragma unroll
@@ -1157,6 +1520,11 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             const int i = tid + e * 256, d = i % dpad;
             if (i >= nt * dpad) continue;
             const bool in = d < p.dim;                  // rows beyond the key size: zero keys, no removal, state stays zero
+            if constexpr (CHANNEL) {
+                const float g = in ? expf(-p.rate[h] * hy_softplus(fz[e])) : 1.f;
+                r_s[i] = fr[e]; w_s[i] = g; u_s[i] = g * fk[e]; b_s[i] = in ? hy_sigmoid(fa[e]) * fk[e] : 0.f;
+                continue;
+            }
             r_s[i] = fr[e]; k_s[i] = fk[e];
             b_s[i] = in ? hy_sigmoid(fa[e]) : 0.f;
             w_s[i] = in ? expf(-p.decay_mult * hy_sigmoid(fz[e])) : 1.f;
@@ -1167,7 +1535,7 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             if (i < nt * CW) v_s[i] = fv[e];
         }
         __syncthreads();
-        {                                             // |k|^2 of a token's head: sixteen neighbouring lanes per token (TOK <= 16 tokens, 256 threads)
+        if constexpr (!CHANNEL) {                     // |k|^2 of a token's head: sixteen neighbouring lanes per token (TOK <= 16 tokens, 256 threads)
             const int t = tid >> 4, l = tid & 15;
             float ss = 0.f;
             if (t < nt)
@@ -1175,15 +1543,17 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             ss = hy_sum16(ss);
             if (t < nt && l == 0) inv_s[t] = 1.f / sqrtf(ss + p.unit_eps);
         }
-        __syncthreads();
+        if constexpr (!CHANNEL) {
+            __syncthreads();
 #pragma unroll
-        for (int e = 0; e < EL; ++e) {
-            const int i = tid + e * 256;
-            if (i >= nt * dpad) continue;
-            const float u = k_s[i] * inv_s[i / dpad];
-            u_s[i] = u; b_s[i] = b_s[i] * u;
+            for (int e = 0; e < EL; ++e) {
+                const int i = tid + e * 256;
+                if (i >= nt * dpad) continue;
+                const float u = k_s[i] * inv_s[i / dpad];
+                u_s[i] = u; b_s[i] = b_s[i] * u;
+            }
+            __syncthreads();
         }
-        __syncthreads();
         if (t0 + TOK < r1) fetch(t0 + TOK);          // in flight during the walk
         // the gates of token t + 1 are read from LDS while token t is worked on (two register sets, taken in turns)
         struct Gates { f32x4 u[RD / 4], w[RD / 4], b[RD / 4], k[RD / 4], r[RD / 4]; float v; };
@@ -1192,7 +1562,8 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
 #pragma unroll
             for (int j4 = 0; j4 < RD / 4; ++j4) {
                 g.u[j4] = *(const f32x4*)(u_s + o + j4 * 4); g.w[j4] = *(const f32x4*)(w_s + o + j4 * 4); g.b[j4] = *(const f32x4*)(b_s + o + j4 * 4);
-                g.k[j4] = *(const f32x4*)(k_s + o + j4 * 4); g.r[j4] = *(const f32x4*)(r_s + o + j4 * 4);
+                if constexpr (!CHANNEL) g.k[j4] = *(const f32x4*)(k_s + o + j4 * 4);
+                g.r[j4] = *(const f32x4*)(r_s + o + j4 * 4);
             }
             g.v = v_s[t * CW + col];
         };
@@ -1210,7 +1581,8 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int j = j4 * 4 + e;
-                    S[j] = __builtin_fmaf(g.w[j4][e], S[j], __builtin_fmaf(-g.b[j4][e], sb, g.k[j4][e] * g.v));
+                    if constexpr (CHANNEL) S[j] = __builtin_fmaf(g.w[j4][e], S[j], g.b[j4][e] * (g.v - sb));
+                    else S[j] = __builtin_fmaf(g.w[j4][e], S[j], __builtin_fmaf(-g.b[j4][e], sb, g.k[j4][e] * g.v));
                     op[e] = __builtin_fmaf(g.r[j4][e], S[j], op[e]);
                 }
             }
@@ -1240,19 +1612,25 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             if (d < p.dim) st[(size_t)d * p.vdim] = S[j];
         }
     }
+    if constexpr (CHANNEL) {
+        if (p.hist && p.taps > 1)
+            hy_conv_advance(p.raw, p.ldr, p.C, p.taps, p.hist + (size_t)p.slot[sq] * (p.taps - 1) * p.C, r0, r1, p.first_pos[sq],
+                            (h * gridDim.z + blockIdx.z) * 256 + tid, p.H * gridDim.z * 256);
+    }
 }
 
 // per-head RMS norm over vdim with a plain weight (null: none; shared by the heads, or w_heads: one per head and channel, [H * vdim]), optional
-// gate (silu, or gate_sigmoid: sigmoid): one block per (row, head), a single wave for heads of up to 256 channels and a wave per 256 channels
+// gate (silu, or gate_sigmoid: sigmoid); den non-null: the head is divided by den[row * H + h] first: one block per (row, head), a single wave for heads of up to 256 channels and a wave per 256 channels
 // beyond, up to sixteen (one "head" that spans all heads of a row: a norm over the whole concatenation)
 template <typename T>
 __global__ __launch_bounds__(1024) void hy_head_norm_kernel(const float* o, int H, int vdim, const T* w, float eps, const float* gate, int ldg, int goff, T* out,
-                                                           int w_heads, int gate_sigmoid) {
+                                                           int w_heads, int gate_sigmoid, const float* den) {
     __shared__ float red[16];
     const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, NT = blockDim.x;
     const float* src = o + ((size_t)r * H + h) * vdim;
+    const float sc = den ? 1.f / den[(size_t)r * H + h] : 1.f;
     float ss = 0.f;
-    for (int c = tid; c < vdim; c += NT) ss = __builtin_fmaf(src[c], src[c], ss);
+    for (int c = tid; c < vdim; c += NT) { const float v = src[c] * sc; ss = __builtin_fmaf(v, v, ss); }
     ss = hy_wave_sum(ss);
     if (NT > 64) {
         if ((tid & 63) == 0) red[tid >> 6] = ss;
@@ -1262,7 +1640,7 @@ __global__ __launch_bounds__(1024) void hy_head_norm_kernel(const float* o, int 
     }
     const float inv = 1.f / sqrtf(ss / (float)vdim + eps);
     for (int c = tid; c < vdim; c += NT) {
-        float v = src[c] * inv;
+        float v = src[c] * sc * inv;
         if (w) v *= (float)w[w_heads ? h * vdim + c : c];
         if (gate) { const float gz = gate[(size_t)r * ldg + goff + h * vdim + c]; v *= gate_sigmoid ? hy_sigmoid(gz) : hy_silu(gz); }
         out[((size_t)r * H + h) * vdim + c] = (T)v;
@@ -1413,15 +1791,15 @@ __device__ __forceinline__ void hy_wave_argmax(float& v, int& i) {
     }
 }
 
-// How a router scores: softmax over the logits or a sigmoid of each (sigmoid != 0); a group's score is its best expert's or the sum of its two
+// How a router scores: score 0 softmax over the logits, 1 a sigmoid of each, 2 softmax over the CHOSEN logits only; a group's score is its best expert's or the sum of its two
 // best (group_top = 1 | 2); the chosen experts weigh score * wscale.
-struct RouteMode { int sigmoid; int group_top; float wscale; };
+struct RouteMode { int score; int group_top; float wscale; };
 
 // The routing of one token by one wave; sc [E] and gb [groups] are the wave's scratch in LDS.  Every thread of the block calls it the same
 // number of times (it holds block barriers); a wave without a token passes active = false.
 __device__ __forceinline__ void hy_route_token(bool active, const float* zr, float* sc, float* gb, int E, int groups, int keep, int top, int32_t* ids,
                                                float* wts, int lane, RouteMode rm) {
-    if (rm.sigmoid) {
+    if (rm.score == 1) {
         if (active) for (int e = lane; e < E; e += 64) sc[e] = hy_sigmoid(zr[e]);
     } else {
         float m = -INFINITY;
@@ -1430,7 +1808,7 @@ __device__ __forceinline__ void hy_route_token(bool active, const float* zr, flo
         float sum = 0.f;
         if (active) for (int e = lane; e < E; e += 64) { const float x = expf(zr[e] - m); sc[e] = x; sum += x; }
         sum = hy_wave_sum(sum);
-        if (active) for (int e = lane; e < E; e += 64) sc[e] = sc[e] / sum;
+        if (active && rm.score == 0) for (int e = lane; e < E; e += 64) sc[e] = sc[e] / sum;     // score 2: e^(z - max), normalised over the chosen below
     }
     __syncthreads();
     const int per = E / groups;
@@ -1456,18 +1834,22 @@ __device__ __forceinline__ void hy_route_token(bool active, const float* zr, flo
         if (active) for (int g = lane; g < groups; g += 64) gb[g] = INFINITY;
         __syncthreads();
     }
-    // sigmoid scores are ranked by their logits (the same order, and it survives where the fp32 sigmoid rounds to one)
+    // sigmoid scores are ranked by their logits (the same order, and it survives where the fp32 sigmoid rounds to one); so are those of score 2, whose
+    // exponentials may underflow
+    float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
         float bv = -INFINITY; int bi = 0x7fffffff;
         if (active)
             for (int e = lane; e < E; e += 64) {
-                const float v = rm.sigmoid ? zr[e] : sc[e];
+                const float v = rm.score ? zr[e] : sc[e];
                 if (sc[e] >= 0.f && gb[e / per] == INFINITY && (bi == 0x7fffffff || v > bv || (v == bv && e < bi))) { bv = v; bi = e; }
             }
         hy_wave_argmax(bv, bi);
-        if (active && lane == 0) { ids[k] = bi; wts[k] = sc[bi] * rm.wscale; sc[bi] = -1.f; }     // taken
+        if (active && lane == 0) { ids[k] = bi; wts[k] = sc[bi] * rm.wscale; chosen += sc[bi]; sc[bi] = -1.f; }     // taken
         __syncthreads();
     }
+    if (rm.score == 2 && active && lane == 0)
+        for (int k = 0; k < top; ++k) wts[k] = wts[k] / chosen;
 }
 
 __global__ __launch_bounds__(64) void hy_moe_route_kernel(const float* z, int ld, int E, int groups, int keep, int top, int32_t* ids, float* wts, RouteMode rm) {
@@ -1535,6 +1917,18 @@ __global__ __launch_bounds__(256) void hy_moe_combine_kernel(const float* y, int
         if (extra) a += extra[(size_t)t * W + c];
         out[(size_t)t * W + c] = a;
     }
+}
+
+// sixteen lanes per value column (16 columns per block) for heads of more than 32 key channels, four (64 columns per block) below
+template <bool CHANNEL>
+void launch_delta(const DeltaParams& p, int nseq, hipStream_t st) {
+    const dim3 g16(nseq, p.H, (p.vdim + 15) / 16), g4(nseq, p.H, (p.vdim + 63) / 64);
+    if (p.dim <= 16)       hipLaunchKernelGGL((hy_delta_kernel<4, 4, CHANNEL>), g4, dim3(256), 0, st, p);
+    else if (p.dim <= 32)  hipLaunchKernelGGL((hy_delta_kernel<8, 4, CHANNEL>), g4, dim3(256), 0, st, p);
+    else if (p.dim <= 64)  hipLaunchKernelGGL((hy_delta_kernel<4, 16, CHANNEL>), g16, dim3(256), 0, st, p);
+    else if (p.dim <= 128) hipLaunchKernelGGL((hy_delta_kernel<8, 16, CHANNEL>), g16, dim3(256), 0, st, p);
+    else if (p.dim <= 192) hipLaunchKernelGGL((hy_delta_kernel<12, 16, CHANNEL>), g16, dim3(256), 0, st, p);
+    else                   hipLaunchKernelGGL((hy_delta_kernel<16, 16, CHANNEL>), g16, dim3(256), 0, st, p);
 }
 
 int hy_geom_ok(const AttnGeom& g) {
@@ -1642,6 +2036,38 @@ extern "C" int mi355_hy_branch_norm(float* x, const float* a, float ca, const fl
     return MI355_OK;
 }
 
+// X fp32 [*, S, W] residual streams, updated in place and read into h [n, W] of act_dtype (see hy_streams_kernel).  terms: y = ca * a + cb * b + mixture sum,
+// a / b fp32 [*, W] or null, normed over the row first under na / nb (act_dtype [W], or null) with neps.  mix fp32 [S, S] ([from, to]) and wr fp32 [S] on the
+// device (mix null: the streams stay as they are and there is no result to add); rd fp32 [S] (null: the sum of the streams).  ids non-null: the streams
+// start as rows of table [vocab, W].  rows: null, or n row indices to form without writing X.  S <= 16.
+extern "C" int mi355_hy_streams(float* X, int32_t n, int32_t S, int32_t W, const float* a, float ca, const void* na, const float* b, float cb, const void* nb, float neps,
+                                const float* moe_y, const int32_t* moe_place, const float* moe_wts, int32_t moe_top, const float* mix, const float* wr, const float* rd,
+                                const int32_t* ids, const void* table, int32_t vocab, const int32_t* rows, const void* w, float eps, void* h, int32_t act_dtype,
+                                mi355_stream_t stream) {
+    MI355_CHECK_ARG(X && n > 0 && S > 0 && S <= 16 && W > 0, "hy_streams: n=%d streams=%d W=%d", n, S, W);
+    MI355_CHECK_ARG((!h || w) && (h || !rows), "hy_streams: a norm needs its weight, gathered rows need an output");
+    MI355_CHECK_ARG(!ids || (table && vocab > 0 && !mix && !a && !b && !moe_y), "hy_streams: the start has no result to add");
+    MI355_CHECK_ARG(!mix || (wr && (a || b || moe_y)), "hy_streams: a write-back needs its result");
+    MI355_CHECK_ARG(mix || !(a || b || moe_y), "hy_streams: a result without the mix of the streams");
+    MI355_CHECK_ARG((!na || a) && (!nb || b), "hy_streams: the norm of an absent branch");
+    MI355_CHECK_ARG(!moe_y || (moe_place && moe_wts && moe_top > 0), "hy_streams: a mixture's sum needs its places and weights");
+    MI355_CHECK_ARG((size_t)W * 4 <= 64 * 1024, "hy_streams: W=%d too wide for one block", W);
+    const StreamTerms st{a, ca, na, b, cb, nb, neps};
+    const MoeSum ms{moe_y, moe_place, moe_wts, moe_top};
+    const StreamMix sm{mix, wr, rd, S};
+    auto al = [](const void* p_) { return ((uintptr_t)p_ & 15) == 0; };
+    const bool vec = W % 4 == 0 && al(X) && al(a) && al(b) && al(na) && al(nb) && al(moe_y) && al(table) && al(w) && al(h);
+    hipStream_t s_ = (hipStream_t)stream;
+#define HY_STREAMS(VEC_, SM_)                                                                                                                                        \
+    HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_streams_kernel<T, VEC_, SM_>), dim3(n), dim3(256), (size_t)W * 4, s_, X, st, ms, sm, ids, (const T*)table, vocab, rows, \
+                                              (const T*)w, eps, W, (T*)h))
+    if (vec) { if (S == 1) HY_STREAMS(true, 1); else if (S == 2) HY_STREAMS(true, 2); else if (S <= 4) HY_STREAMS(true, 4); else if (S <= 8) HY_STREAMS(true, 8); else HY_STREAMS(true, 16); }
+    else     { if (S <= 2) HY_STREAMS(false, 2); else if (S <= 4) HY_STREAMS(false, 4); else HY_STREAMS(false, 16); }
+#undef HY_STREAMS
+    MI355_CHECK_LAUNCH("hy_streams_kernel");
+    return MI355_OK;
+}
+
 // x fp32 [T, W] stream (the layer's input plus its earlier branches), a fp32 [T, W] or null; stack fp32 [>= n + 1, T, W] with planes 0 .. n - 1 filled;
 // coef fp32 [n + 1] on the device.  Writes stack[n] = x + a, x = sum_j coef[j] stack[j], h1 [rows_n, W] of act_dtype (null: no norm).  rows: null
 // (rows_n = T rows, in place), or rows_n row indices to form without writing x or the stack.
@@ -1718,8 +2144,18 @@ extern "C" int mi355_hy_attn_rows_ex(const float* q, int32_t ldq, float scale, c
                                      const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache,
                                      const void* vcache, void* out, int32_t splits, float* parts, int32_t window, float softcap, const float* ogate,
                                      int32_t ldg, int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0]), "hy_attn_rows: window=%d chunk=%d ldg=%d", window, chunk, ldg);
-    const AttnExtra ex{window, softcap, ogate, ldg};
+    return mi355_hy_attn_rows_ex2(q, ldq, scale, geom, chunk, sink, vfreq, pos, seq, block_table, rows, kcache, vcache, out, splits, parts, window, softcap, ogate, ldg, 0,
+                                  act_dtype, stream);
+}
+
+// gate_channels != 0: ogate holds one pre-activation per value channel (fp32 [rows, ldg], column h * vdim + c) instead of one per head.
+extern "C" int mi355_hy_attn_rows_ex2(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                                      const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache,
+                                      const void* vcache, void* out, int32_t splits, float* parts, int32_t window, float softcap, const float* ogate,
+                                      int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(geom && window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
+                    "hy_attn_rows: window=%d chunk=%d ldg=%d", window, chunk, ldg);
+    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels};
     MI355_CHECK_ARG(q && geom && pos && seq && block_table && kcache && vcache && out && rows > 0 && chunk >= 0, "hy_attn_rows: bad argument");
     MI355_CHECK_ARG(splits >= 1 && splits <= 64 && (splits == 1 || parts), "hy_attn_rows: %d splits", splits);
     MI355_CHECK_ARG(!vfreq || geom[3] % 2 == 0, "hy_attn_rows: rotated values need an even value size (%d)", geom[3]);
@@ -1750,8 +2186,17 @@ extern "C" int mi355_hy_attn_tiles_ex(const float* q, int32_t ldq, float scale, 
                                       const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0,
                                       const int32_t* tile_n, int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, float softcap,
                                       const float* ogate, int32_t ldg, int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0]), "hy_attn_tiles: window=%d chunk=%d ldg=%d", window, chunk, ldg);
-    const AttnExtra ex{window, softcap, ogate, ldg};
+    return mi355_hy_attn_tiles_ex2(q, ldq, scale, geom, chunk, sink, vfreq, pos, seq, block_table, tile_row0, tile_n, tiles, kcache, vcache, out, window, softcap, ogate,
+                                   ldg, 0, act_dtype, stream);
+}
+
+extern "C" int mi355_hy_attn_tiles_ex2(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                                       const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0,
+                                       const int32_t* tile_n, int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, float softcap,
+                                       const float* ogate, int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(geom && window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
+                    "hy_attn_tiles: window=%d chunk=%d ldg=%d", window, chunk, ldg);
+    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels};
     MI355_CHECK_ARG(q && geom && pos && seq && block_table && tile_row0 && tile_n && kcache && vcache && out && tiles > 0 && chunk >= 0, "hy_attn_tiles: bad argument");
     const AttnGeom g{geom[0], geom[1], geom[2], geom[3], geom[4], geom[5], geom[6], geom[7], geom[8], geom[9], geom[10] > 0 ? geom[10] : geom[3]};
     if (int e = hy_geom_ok(g)) return e;
@@ -1794,13 +2239,67 @@ extern "C" int mi355_hy_scan(int32_t mode, const float* proj, int32_t ld, int32_
     int tok = 16;                                                // staged tokens: keep the LDS buffers under 60 KiB
     auto lds_of = [&](int t) { return (size_t)(3 * t * DS * RD + t * 64 + t * DS * 64) * 4; };
     while (tok > 1 && lds_of(tok) > 60 * 1024) tok >>= 1;
-    ScanParams p{proj, ld, qo, ko, vo, z, ldz, lower, fbias, tau, qscale, mode & 3, H, dim, vdim, row_start, slot, first_pos, state, out, tok, (mode & 4) ? 1 : 0};
+    ScanParams p{proj, ld, qo, ko, vo, z, ldz, lower, fbias, tau, qscale, mode & 3, H, dim, vdim, row_start, slot, first_pos, state, out, tok, (mode & 4) ? 1 : 0, {}};
     const size_t lds = lds_of(tok);
     const dim3 grid(nseq, H, (vdim + 63) / 64);
     if (RD == 8)       HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_scan_kernel<T, 8>), grid, dim3(64 * DS), lds, (hipStream_t)stream, p));
     else if (RD == 16) HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_scan_kernel<T, 16>), grid, dim3(64 * DS), lds, (hipStream_t)stream, p));
     else               HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_scan_kernel<T, 32>), grid, dim3(64 * DS), lds, (hipStream_t)stream, p));
     MI355_CHECK_LAUNCH("hy_scan_kernel");
+    return MI355_OK;
+}
+
+// Matrix memory under exponential gates.  proj fp32 [rows, ld]: q, k (H heads of dim), v (H heads of vdim) at columns qo, ko, vo, pre-activations of the input
+// and forget gates (H each, biases included) at io, fo; both pass cap tanh(z / cap).  state fp32 [slots, H, dim * vdim + dim] (S, then n), mstate fp32
+// [slots, H, nz] with nz = ceil(vdim / 64) (copies of the running maximum).  out fp32 [rows, H * vdim] = S^T (qscale q), den fp32 [rows, H].
+// pass 0: the walk.  The chunked form: mi355_hy_memory_gates, then pass 1 over the chunks as sequences from zero states (cdecay fp32 [chunks, H] receives their
+// total decays, den the bare n . q), mi355_hy_chunk_prefix_ex, and pass 2 (states read only, out and den completed); gates fp32 [rows, H, 3] in both.
+extern "C" int mi355_hy_memory_scan(int32_t pass, const float* proj, int32_t ld, int32_t qo, int32_t ko, int32_t vo, int32_t io, int32_t fo, float cap, float qscale,
+                                    float den_eps, int32_t H, int32_t dim, int32_t vdim, const int32_t* row_start, const int32_t* slot, const int32_t* first_pos,
+                                    int32_t nseq, float* state, float* mstate, const float* gates, float* cdecay, float* den, float* out, mi355_stream_t stream) {
+    MI355_CHECK_ARG(proj && row_start && slot && first_pos && state && den && out && nseq > 0 && H > 0 && dim > 0 && vdim > 0, "hy_memory_scan: bad argument");
+    MI355_CHECK_ARG(pass >= 0 && pass <= 2 && (pass == 0 ? (mstate && !gates) : gates != nullptr) && (pass != 1 || cdecay), "hy_memory_scan: pass %d lacks its inputs", pass);
+    MI355_CHECK_ARG(dim <= 512 && cap > 0.f, "hy_memory_scan: key size %d (<= 512), gate cap %g", dim, (double)cap);
+    const int RD = dim <= 128 ? 8 : dim <= 256 ? 16 : 32;
+    const int DS = (dim + RD - 1) / RD;
+    int tok = 16;
+    auto lds_of = [&](int t) { return (size_t)(3 * t * DS * RD + t * 64 + t * DS * 64) * 4; };
+    while (tok > 1 && lds_of(tok) > 60 * 1024) tok >>= 1;
+    const dim3 grid(nseq, H, (vdim + 63) / 64);
+    ScanParams p{proj, ld, qo, ko, vo, nullptr, 0, nullptr, nullptr, 1.f, qscale, SCAN_FIXED, H, dim, vdim, row_start, slot, first_pos, state, out, tok, pass == 2 ? 1 : 0,
+                 MemGates{io, fo, cap, den_eps, pass ? gates : nullptr, mstate, (int)grid.z, pass == 1 ? cdecay : nullptr, den, pass == 1 ? 1 : 0}};
+    const size_t lds = lds_of(tok);
+    hipStream_t st = (hipStream_t)stream;
+    if (RD == 8)       hipLaunchKernelGGL((hy_scan_kernel<float, 8, true>), grid, dim3(64 * DS), lds, st, p);
+    else if (RD == 16) hipLaunchKernelGGL((hy_scan_kernel<float, 16, true>), grid, dim3(64 * DS), lds, st, p);
+    else               hipLaunchKernelGGL((hy_scan_kernel<float, 32, true>), grid, dim3(64 * DS), lds, st, p);
+    MI355_CHECK_LAUNCH("hy_memory_scan");
+    return MI355_OK;
+}
+
+// The gates of every row for the chunked form: out fp32 [rows, H, 3] = keep, take, e^(-m); mstate is continued and left at the sequences' ends.
+extern "C" int mi355_hy_memory_gates(const float* proj, int32_t ld, int32_t io, int32_t fo, float cap, int32_t H, const int32_t* row_start, const int32_t* slot,
+                                     const int32_t* first_pos, int32_t nseq, float* mstate, int32_t nz, float* out, mi355_stream_t stream) {
+    MI355_CHECK_ARG(proj && row_start && slot && first_pos && mstate && out && nseq > 0 && H > 0 && nz > 0 && nz <= 1024 && cap > 0.f, "hy_memory_gates: bad argument");
+    const MemGates g{io, fo, cap, 0.f, nullptr, mstate, nz, nullptr, nullptr, 0};
+    hipLaunchKernelGGL(hy_memory_gates_kernel, dim3(nseq, H), dim3(1024), 0, (hipStream_t)stream, proj, ld, g, H, row_start, slot, first_pos, out);
+    MI355_CHECK_LAUNCH("hy_memory_gates_kernel");
+    return MI355_OK;
+}
+
+// Short causal convolutions + silu + unit heads (see hy_short_conv_kernel): proj fp32 [rows, ld], channels 0 .. C - 1 convolved under w [C, taps] of act_dtype,
+// the first `units` heads of dim channels brought to unit length (the first uq of them times qscale); hist fp32 [slots, taps - 1, C] is read; out fp32 [rows, C].
+// low non-null: columns lo .. lo + R - 1 rounded to act_dtype [rows, R].
+extern "C" int mi355_hy_short_conv(const float* proj, int32_t ld, int32_t rows, int32_t C, int32_t taps, const void* w, int32_t units, int32_t uq, int32_t dim,
+                                   float qscale, float unit_eps, const float* hist, const int32_t* seq, const int32_t* row_start, const int32_t* slot,
+                                   const int32_t* first_pos, float* out, int32_t lo, int32_t R, void* low, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(proj && w && seq && row_start && slot && first_pos && out && rows > 0 && C > 0 && taps > 0 && (hist || taps == 1), "hy_short_conv: bad argument");
+    MI355_CHECK_ARG(units >= 0 && uq >= 0 && uq <= units && units * dim <= C && (units == 0 || (dim > 0 && dim <= 512)), "hy_short_conv: %d heads of %d in %d channels", units, dim, C);
+    MI355_CHECK_ARG(ld >= C && (!low || (R > 0 && lo >= 0 && ld >= lo + R)), "hy_short_conv: ld=%d lo=%d R=%d", ld, lo, R);
+    const ConvParams p{proj, ld, C, taps, w, units, uq, dim, qscale, unit_eps, hist, seq, row_start, slot, first_pos, out, lo, R, low};
+    const int pv = (C - units * dim + CONV_PIECE - 1) / CONV_PIECE, pieces = units + pv + (low ? (R + CONV_PIECE - 1) / CONV_PIECE : 0);
+    HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_short_conv_kernel<T>, dim3(rows, (pieces + 3) / 4), dim3(256), 0, (hipStream_t)stream, p, pv, pieces));
+    MI355_CHECK_LAUNCH("hy_short_conv_kernel");
     return MI355_OK;
 }
 
@@ -1818,9 +2317,15 @@ extern "C" int mi355_hy_chunk_plan(const int32_t* row_start, int32_t nseq, int32
 // state [slots, H, dim * vdim] is continued (from zero where first_pos is 0) and receives the sequences' final states.  decay fp32 [H].
 extern "C" int mi355_hy_chunk_prefix(const int32_t* cs, const int32_t* sc, const int32_t* slot, const int32_t* first_pos, int32_t nseq, const float* decay, int32_t H,
                                      int32_t per_head, float* chunk_state, float* state, mi355_stream_t stream) {
-    MI355_CHECK_ARG(cs && sc && slot && first_pos && decay && chunk_state && state && nseq > 0 && H > 0 && per_head > 0, "hy_chunk_prefix: nseq=%d H=%d", nseq, H);
+    return mi355_hy_chunk_prefix_ex(cs, sc, slot, first_pos, nseq, decay, nullptr, H, per_head, chunk_state, state, stream);
+}
+
+// cdecay non-null (fp32 [chunks, H]): the total decay of every chunk, where the decay is not one constant per head (decay may be null then).
+extern "C" int mi355_hy_chunk_prefix_ex(const int32_t* cs, const int32_t* sc, const int32_t* slot, const int32_t* first_pos, int32_t nseq, const float* decay,
+                                        const float* cdecay, int32_t H, int32_t per_head, float* chunk_state, float* state, mi355_stream_t stream) {
+    MI355_CHECK_ARG(cs && sc && slot && first_pos && (decay || cdecay) && chunk_state && state && nseq > 0 && H > 0 && per_head > 0, "hy_chunk_prefix: nseq=%d H=%d", nseq, H);
     hipLaunchKernelGGL(hy_chunk_prefix_kernel, dim3(nseq, H, (per_head + 255) / 256), dim3(256), 0, (hipStream_t)stream, cs, sc, slot, first_pos, decay, H, per_head,
-                       chunk_state, state);
+                       chunk_state, state, cdecay);
     MI355_CHECK_LAUNCH("hy_chunk_prefix_kernel");
     return MI355_OK;
 }
@@ -1834,16 +2339,29 @@ extern "C" int mi355_hy_delta_scan(const float* proj, int32_t ld, int32_t ro, in
     MI355_CHECK_ARG(proj && z && row_start && slot && first_pos && state && out && nseq > 0 && H > 0 && dim > 0 && vdim > 0, "hy_delta_scan: bad argument");
     MI355_CHECK_ARG(dim <= 256, "hy_delta_scan: key size %d > 256", dim);
     MI355_CHECK_ARG(ld >= H * dim && ldz >= H * dim && unit_eps >= 0.f, "hy_delta_scan: ld=%d ldz=%d", ld, ldz);
-    DeltaParams p{proj, ld, ro, ko, vo, ao, z, ldz, decay_mult, unit_eps, H, dim, vdim, row_start, slot, first_pos, state, out};
-    hipStream_t st = (hipStream_t)stream;
-    // sixteen lanes per value column (16 columns per block) for heads of more than 32 key channels, four (64 columns per block) below
-    const dim3 g16(nseq, H, (vdim + 15) / 16), g4(nseq, H, (vdim + 63) / 64);
-    if (dim <= 16)       hipLaunchKernelGGL((hy_delta_kernel<4, 4>), g4, dim3(256), 0, st, p);
-    else if (dim <= 32)  hipLaunchKernelGGL((hy_delta_kernel<8, 4>), g4, dim3(256), 0, st, p);
-    else if (dim <= 64)  hipLaunchKernelGGL((hy_delta_kernel<4, 16>), g16, dim3(256), 0, st, p);
-    else if (dim <= 128) hipLaunchKernelGGL((hy_delta_kernel<8, 16>), g16, dim3(256), 0, st, p);
-    else if (dim <= 192) hipLaunchKernelGGL((hy_delta_kernel<12, 16>), g16, dim3(256), 0, st, p);
-    else                 hipLaunchKernelGGL((hy_delta_kernel<16, 16>), g16, dim3(256), 0, st, p);
+    DeltaParams p{};
+    p.proj = proj; p.ld = ld; p.ro = ro; p.ko = ko; p.vo = vo; p.ao = ao; p.z = z; p.ldz = ldz; p.decay_mult = decay_mult; p.unit_eps = unit_eps;
+    p.H = p.G = H; p.dim = dim; p.vdim = vdim; p.row_start = row_start; p.slot = slot; p.first_pos = first_pos; p.state = state; p.out = out;
+    launch_delta<false>(p, nseq, (hipStream_t)stream);
+    MI355_CHECK_LAUNCH("hy_delta_kernel");
+    return MI355_OK;
+}
+
+// The delta rule with a decay per key channel (CHANNEL instances of hy_delta_kernel).  x fp32 [rows, ld]: r (G heads of dim), k (G heads of dim), v (H heads of
+// vdim) at columns ro, ko, vo, ready for the recurrence; z fp32 [rows, ldz] + zbias fp32 [H * dim]: decay pre-activation; rate fp32 [H]; bp fp32 [rows, ldb]: one
+// step-size pre-activation per head.  hist non-null: the short convolution's state fp32 [slots, taps - 1, C] is moved on from its raw inputs raw [rows, ldr].
+extern "C" int mi355_hy_channel_delta_scan(const float* x, int32_t ld, int32_t ro, int32_t ko, int32_t vo, const float* z, int32_t ldz, const float* zbias,
+                                           const float* rate, const float* bp, int32_t ldb, int32_t H, int32_t G, int32_t dim, int32_t vdim,
+                                           const int32_t* row_start, const int32_t* slot, const int32_t* first_pos, int32_t nseq, float* state, float* out,
+                                           const float* raw, int32_t ldr, int32_t C, int32_t taps, float* hist, mi355_stream_t stream) {
+    MI355_CHECK_ARG(x && z && zbias && rate && bp && row_start && slot && first_pos && state && out && nseq > 0 && H > 0 && dim > 0 && vdim > 0, "hy_channel_delta_scan: bad argument");
+    MI355_CHECK_ARG(G > 0 && H % G == 0 && dim <= 256, "hy_channel_delta_scan: %d heads over %d key heads of %d (<= 256)", H, G, dim);
+    MI355_CHECK_ARG(ldz >= H * dim && ldb >= H && ld >= 2 * G * dim + H * vdim && (!hist || (raw && ldr >= C && C > 0 && taps > 0)), "hy_channel_delta_scan: ld=%d ldz=%d ldb=%d", ld, ldz, ldb);
+    DeltaParams p{};
+    p.proj = x; p.ld = ld; p.ro = ro; p.ko = ko; p.vo = vo; p.z = z; p.ldz = ldz; p.zbias = zbias; p.rate = rate; p.bp = bp; p.ldb = ldb;
+    p.H = H; p.G = G; p.dim = dim; p.vdim = vdim; p.row_start = row_start; p.slot = slot; p.first_pos = first_pos; p.state = state; p.out = out;
+    p.raw = raw; p.ldr = ldr; p.C = C; p.taps = taps; p.hist = hist;
+    launch_delta<true>(p, nseq, (hipStream_t)stream);
     MI355_CHECK_LAUNCH("hy_delta_kernel");
     return MI355_OK;
 }
@@ -1856,9 +2374,16 @@ extern "C" int mi355_hy_head_norm(const float* o, int32_t rows, int32_t H, int32
 // w_heads: w is [H * vdim] (a weight per head and channel) instead of [vdim]; gate_sigmoid: the gate is sigmoid(gate) instead of silu(gate).
 extern "C" int mi355_hy_head_norm_ex(const float* o, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg,
                                      int32_t goff, void* out, int32_t w_heads, int32_t gate_sigmoid, int32_t act_dtype, mi355_stream_t stream) {
+    return mi355_hy_head_norm_ex2(o, rows, H, vdim, w, eps, gate, ldg, goff, out, w_heads, gate_sigmoid, nullptr, act_dtype, stream);
+}
+
+// den: null, or fp32 [rows, H]: head h of a row is divided by den[row, h] before its norm.
+extern "C" int mi355_hy_head_norm_ex2(const float* o, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg,
+                                      int32_t goff, void* out, int32_t w_heads, int32_t gate_sigmoid, const float* den, int32_t act_dtype,
+                                      mi355_stream_t stream) {
     MI355_CHECK_ARG(o && out && rows > 0 && H > 0 && vdim > 0, "hy_head_norm: bad argument");
     HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_head_norm_kernel<T>, dim3(rows, H), dim3(vdim > 256 ? std::min(1024, (vdim + 255) / 256 * 64) : 64), 0, (hipStream_t)stream, o, H, vdim, (const T*)w, eps,
-                                              gate, ldg, goff, (T*)out, w_heads, gate_sigmoid));
+                                              gate, ldg, goff, (T*)out, w_heads, gate_sigmoid, den));
     MI355_CHECK_LAUNCH("hy_head_norm_kernel");
     return MI355_OK;
 }
@@ -1906,12 +2431,13 @@ extern "C" int mi355_hy_moe_route(const float* z, int32_t ld, int32_t tokens, in
     return mi355_hy_moe_route_ex(z, ld, tokens, E, groups, keep, top, ids, wts, 0, 1, 1.f, stream);
 }
 
-// The same with the router's form as arguments: score_sigmoid (scores are sigmoids of the logits instead of their softmax), group_top (1: a group
+// The same with the router's form as arguments: score (0: softmax over all logits, 1: a sigmoid of each, 2: softmax over the chosen ones), group_top (1: a group
 // scores as its best expert; 2: as the sum of its two best), wscale (the chosen experts weigh score * wscale).
 extern "C" int mi355_hy_moe_route_ex(const float* z, int32_t ld, int32_t tokens, int32_t E, int32_t groups, int32_t keep, int32_t top, int32_t* ids, float* wts,
-                                     int32_t score_sigmoid, int32_t group_top, float wscale, mi355_stream_t stream) {
+                                     int32_t score, int32_t group_top, float wscale, mi355_stream_t stream) {
+    MI355_CHECK_ARG(score >= 0 && score <= 2, "hy_moe_route: score form %d", score);
     MI355_CHECK_ARG(group_top == 1 || group_top == 2, "hy_moe_route: a group scores by its best %d experts (1 or 2)", group_top);
-    const RouteMode rm{score_sigmoid, group_top, wscale};
+    const RouteMode rm{score, group_top, wscale};
     MI355_CHECK_ARG(z && ids && wts && tokens > 0 && E > 0 && ld >= E, "hy_moe_route: tokens=%d experts=%d", tokens, E);
     MI355_CHECK_ARG(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top >= 1 && top <= (E / groups) * keep, "hy_moe_route: %d experts in %d groups, keep %d, top %d",
                     E, groups, keep, top);
@@ -1937,10 +2463,11 @@ extern "C" int mi355_hy_moe_route_align(const float* z, int32_t ld, int32_t toke
 }
 
 extern "C" int mi355_hy_moe_route_align_ex(const float* z, int32_t ld, int32_t tokens, int32_t E, int32_t groups, int32_t keep, int32_t top, int32_t* ids,
-                                           float* wts, int32_t* offs, int32_t* src_row, int32_t* place_of, int32_t* tiles, int32_t score_sigmoid,
+                                           float* wts, int32_t* offs, int32_t* src_row, int32_t* place_of, int32_t* tiles, int32_t score,
                                            int32_t group_top, float wscale, mi355_stream_t stream) {
+    MI355_CHECK_ARG(score >= 0 && score <= 2, "hy_moe_route_align: score form %d", score);
     MI355_CHECK_ARG(group_top == 1 || group_top == 2, "hy_moe_route_align: a group scores by its best %d experts (1 or 2)", group_top);
-    const RouteMode rm{score_sigmoid, group_top, wscale};
+    const RouteMode rm{score, group_top, wscale};
     MI355_CHECK_ARG(z && ids && wts && offs && src_row && place_of && tiles && tokens > 0 && E > 0 && ld >= E, "hy_moe_route_align: tokens=%d experts=%d", tokens, E);
     MI355_CHECK_ARG(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top >= 1 && top <= (E / groups) * keep, "hy_moe_route_align: %d experts in %d groups, keep %d, top %d",
                     E, groups, keep, top);

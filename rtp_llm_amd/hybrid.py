@@ -20,36 +20,43 @@ x <- x + LN(mlp(x)): the sublayers read the stream itself and a layer norm follo
 with a learned sink and queries / keys normed over all heads at once beside lightning attention; mixtures of clamped gated experts under a
 sigmoid router whose groups rank by their two best, with a gated shared expert; the embedding is scaled on entry and is the output head;
 checkpoint tensors l<i>.mix.left.{q, k, v, q.norm, k.norm, sink, o}, l<i>.mix.right.{q, k, v, g, norm, o}, l<i>.mlp.{router, e<j>.*, shared.{gate, up,
-down, sg}})."""
+down, sg}}) and Dupenex (the residual is several parallel streams: a sublayer reads one learned weighted sum of them and its result is written back
+to all while they are mixed with each other (l<i>.hc1 / hc2.{in, out, mix}); a span of layers may run several times in a row with the same weights,
+every run with a cache or state of its own; mixers: a delta rule with a decay per key channel behind short convolutions, and windowed attention
+with an elementwise output gate beside a matrix memory under exponential gates, both normed before they are added; silu-gated MLPs and
+mixtures of plain squared-relu experts weighted by the softmax over the chosen logits; checkpoint tensors l<i>.mix.{q, k, v (+ .conv), b, A_log, a1,
+a2, dt_bias, g1, g2, norm, o}, l<i>.mix.left.{q, k, v, g, o, out}, l<i>.mix.right.{q, k, v, g, i, f (+ .b), norm, o, out}, l<i>.mlp.{gate, up, down} or
+l<i>.mlp.{router, e<j>.{up, down}})."""
 import json
 import os
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Union
+from typing import Dict, List, Optional, Tuple, Union
 
 import torch
 
 from . import hybrid_ops as hops
-from .mixers import (AttentionSpec, DeltaRuleSpec, GatedLinearRecurrence, GatedMLP, GeneralizedDeltaRule, LatentAttention, LatentAttentionSpec,
-                     LightningAttention, LightningSpec, PagedChunkAttention, ParallelMixer, PolyNormMLP, RecurrenceSpec, Retention, RetentionSpec,
-                     RotarySpec, RoutedExperts, RouterSpec, StepBatch)
+from .mixers import (AttentionSpec, ChannelDelta, ChannelDeltaSpec, DeltaRuleSpec, GatedLinearRecurrence, GatedMLP, GeneralizedDeltaRule, LatentAttention,
+                     LatentAttentionSpec, LightningAttention, LightningSpec, MatrixMemory, MatrixMemorySpec, PagedChunkAttention, ParallelMixer, PolyNormMLP,
+                     RecurrenceSpec, Retention, RetentionSpec, RotarySpec, RoutedExperts, RouterSpec, StepBatch, state_shapes)
 
 
 @dataclass
 class ParallelSpec:
     """Two mixers on the same input, added as left_scale * left + right_scale * right; their checkpoint tensors sit under mix.left. / mix.right."""
-    left: Union[AttentionSpec, LightningSpec]
-    right: Union[AttentionSpec, LightningSpec]
+    left: Union[AttentionSpec, LightningSpec, MatrixMemorySpec]
+    right: Union[AttentionSpec, LightningSpec, MatrixMemorySpec]
     left_scale: float = 1.0
     right_scale: float = 1.0
+    out_norms: bool = False                          # each side's output is RMS-normed under its own weight (mix.left.out / mix.right.out) first
 
 
 @dataclass
 class HybridLayerSpec:
-    kind: str                                        # "attention" | "hgrn2" | "gla" | "latent_attention" | "retention" | "delta_rule" | "lightning" | "parallel"
-    mixer: Union[AttentionSpec, RecurrenceSpec, LatentAttentionSpec, RetentionSpec, DeltaRuleSpec, LightningSpec, ParallelSpec]
+    kind: str                                        # "attention" | "hgrn2" | "gla" | "latent_attention" | "retention" | "delta_rule" | "channel_delta" | "lightning" | "parallel"
+    mixer: Union[AttentionSpec, RecurrenceSpec, LatentAttentionSpec, RetentionSpec, DeltaRuleSpec, ChannelDeltaSpec, LightningSpec, ParallelSpec]
     ff: Optional[int] = None                         # None: the layer has no MLP; hidden size of the dense MLP or of one routed expert
     mlp_act: str = "relu"
-    mlp_kind: str = "gated"                          # "gated" | "polynorm" | "experts"
+    mlp_kind: str = "gated"                          # "gated" | "polynorm" | "experts" | "plain_experts" (no gate projection: down(act(up h)))
     router: Optional[RouterSpec] = None              # experts: the router ...
     shared_ff: Optional[int] = None                  # ... and the hidden size of the expert every token runs (None: no such expert)
     act_param: float = 0.0                           # parameter of mlp_act (the limit of "swiglu_clamp") ...
@@ -85,7 +92,19 @@ class HybridConfig:
     embed_scale: float = 1.0                         # the embedding rows are multiplied by this as they enter the stream
     tied_head: bool = False                          # the output head is the embedding table itself (without embed_scale); no `head` tensor
     out_norm: bool = False                           # sequential layers whose sublayers read the stream ITSELF and whose OUTPUT is normed: x <- x + norm(f(x))
+    streams: int = 0                                 # > 0: the residual is this many parallel streams mixed at every sublayer (sequential layers)
+    loop: Optional[Tuple[int, int, int]] = None      # (start, stop, times): layers start .. stop - 1 run `times` times in a row with the same weights
     norm_kind: str = "rms"                           # "rms" | "layer" (mean removed, variance of the deviations, a weight and no bias)
+
+    def layer_runs(self) -> List[int]:
+        """Layer indices in the order they run; every entry has a cache or state of its own."""
+        n = len(self.layers)
+        if self.loop is None:
+            return list(range(n))
+        start, stop, times = self.loop
+        if not 0 <= start <= stop <= n or times < 0:
+            raise ValueError(f"loop: layers {start} .. {stop - 1} of {n}, {times} times")
+        return list(range(start)) + list(range(start, stop)) * times + list(range(stop, n))
 
     @staticmethod
     def from_json(cfg: dict) -> "HybridConfig":
@@ -241,7 +260,48 @@ def nudorax_from_json(cfg: dict) -> HybridConfig:
                         embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), tied_head=True)
 
 
-_READERS = {"nufalorn": HybridConfig.nufalorn_from_json, "pokepel": HybridConfig.pokepel_from_json, "nepudra": nepudra_from_json, "nudorax": nudorax_from_json}
+def dupenex_from_json(cfg: dict) -> HybridConfig:
+    """The Dupenex reading of config.json.  Layer types: "channel_delta" (mixer.{heads, kv_heads, dim, vdim, conv}) and "parallel" (mixer.left = windowed
+    attention {heads, kv_heads, dim, vdim, scale, mask.size, rot.{dims, base}} with interleaved rotary pairs and a gate per channel, mixer.right = matrix
+    memory {heads, dim, vdim, gate_cap}; half the sum of both, each normed).  mlp: null, {kind: dense, ff} (silu-gated) or {kind: moe, expert.ff,
+    router.{experts, top}} (squared-relu experts, softmax over the chosen logits).  streams: the residual's streams; loop.{start, stop, times}."""
+    def attention(mx):
+        mask = mx.get("mask") or {}
+        return AttentionSpec(heads=int(mx["heads"]), kv_heads=int(mx.get("kv_heads") or mx["heads"]), dim=int(mx["dim"]), vdim=int(mx.get("vdim") or mx["dim"]),
+                             scale=float(mx["scale"]), rot=RotarySpec.from_json(mx.get("rot"), "interleaved"), window=int(mask.get("size") or 0), out_gate=True,
+                             gate_channels=True)
+
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        kind, mx, mlp = L["type"], L["mixer"], L.get("mlp")
+        if kind == "channel_delta":
+            spec = ChannelDeltaSpec(heads=int(mx["heads"]), kv_heads=int(mx.get("kv_heads") or mx["heads"]), dim=int(mx["dim"]), vdim=int(mx.get("vdim") or mx["dim"]),
+                                    conv=int(mx["conv"]))
+        elif kind == "parallel":
+            b = mx["right"]
+            spec = ParallelSpec(attention(mx["left"]), MatrixMemorySpec(heads=int(b["heads"]), dim=int(b["dim"]), vdim=int(b.get("vdim") or b["dim"]),
+                                                                        gate_cap=float(b["gate_cap"])), 0.5, 0.5, out_norms=True)
+        else:
+            raise NotImplementedError(f"layer {i}: mixer type {kind!r}")
+        if mlp is None:
+            layers.append(HybridLayerSpec(kind, spec))
+        elif mlp.get("kind", "dense") == "dense":
+            layers.append(HybridLayerSpec(kind, spec, int(mlp["ff"]), "silu"))
+        elif mlp["kind"] == "moe":
+            r = mlp["router"]
+            layers.append(HybridLayerSpec(kind, spec, int(mlp["expert"]["ff"]), "relu2", "plain_experts",
+                                          RouterSpec(int(r["experts"]), int(r["top"]), score="softmax_chosen")))
+        else:
+            raise NotImplementedError(f"layer {i}: mlp kind {mlp.get('kind')!r}")
+    loop = cfg.get("loop")
+    c = HybridConfig(name=str(cfg["architecture"]), vocab=int(cfg["vocab"]), width=int(cfg["width"]), layers=layers, eps=float(cfg["norm"]["eps"]), norm_offset=0.0,
+                     sequential=True, streams=int(cfg.get("streams") or 1), loop=(int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else None)
+    c.layer_runs()                                       # the loop's span is checked here
+    return c
+
+
+_READERS = {"nufalorn": HybridConfig.nufalorn_from_json, "pokepel": HybridConfig.pokepel_from_json, "nepudra": nepudra_from_json, "nudorax": nudorax_from_json,
+            "dupenex": dupenex_from_json}
 
 
 class HybridModel:
@@ -297,6 +357,8 @@ class HybridModel:
                 return LightningAttention(a, sub(q, ["q", "k", "v", "g", "norm", "o"]), cfg.eps, self.device)
 
             def side(a, q):
+                if isinstance(a, MatrixMemorySpec):
+                    return MatrixMemory(a, sub(q, ["q", "k", "v", "g", "i", "i.b", "f", "f.b", "norm", "o"]), cfg.eps, self.device)
                 if isinstance(a, AttentionSpec):
                     if a.kv_from is not None:
                         raise NotImplementedError("a side of a parallel mixer keeps its own keys and values")
@@ -308,7 +370,11 @@ class HybridModel:
             elif L.kind == "lightning":
                 mixer = lightning(L.mixer, p + "mix.")
             elif L.kind == "parallel":
-                mixer = ParallelMixer(side(L.mixer.left, p + "mix.left."), side(L.mixer.right, p + "mix.right."), L.mixer.left_scale, L.mixer.right_scale)
+                mixer = ParallelMixer(side(L.mixer.left, p + "mix.left."), side(L.mixer.right, p + "mix.right."), L.mixer.left_scale, L.mixer.right_scale,
+                                      (get(p + "mix.left.out"), get(p + "mix.right.out")) if L.mixer.out_norms else None)
+            elif L.kind == "channel_delta":
+                mixer = ChannelDelta(L.mixer, sub(p + "mix.", ["q", "k", "v", "q.conv", "k.conv", "v.conv", "b", "A_log", "a1", "a2", "dt_bias", "g1", "g2", "norm", "o"]),
+                                     cfg.eps, self.device)
             elif L.kind == "delta_rule":
                 mixer = GeneralizedDeltaRule(L.mixer, sub(p + "mix.", ["r", "k", "v", "a", "a.b", "g", "w1", "w2", "w0", "norm", "o"]), cfg.eps)
             elif L.kind == "latent_attention":
@@ -328,7 +394,7 @@ class HybridModel:
                     mlp = PolyNormMLP(get(p + "mlp.up"), get(p + "mlp.down"), tensors[p + "mlp.act"], cfg.eps)
                 else:
                     ex = [p + f"mlp.e{j}." for j in range(L.router.experts)]
-                    mlp = RoutedExperts(L.router, get(p + "mlp.router"), [get(q + "gate") for q in ex], [get(q + "up") for q in ex],
+                    mlp = RoutedExperts(L.router, get(p + "mlp.router"), None if L.mlp_kind == "plain_experts" else [get(q + "gate") for q in ex], [get(q + "up") for q in ex],
                                         [get(q + "down") for q in ex],
                                         gated(p + "mlp.shared.", L.mlp_act, L.shared_act_param or L.act_param) if L.shared_ff is not None else None, L.mlp_act,
                                         act_param=L.act_param, shared_gate=get(p + "mlp.shared.sg") if L.shared_gate else None)
@@ -355,6 +421,20 @@ class HybridModel:
                 gate_w = torch.cat([mixer.w_in, zrow, gate_w], 0).contiguous()
                 mixer.w_in = None                      # lives on as the leading rows of the shared weight
             self.layers.append((L, mixer, mlp, norm_w(p + "norm1"), n2, gate_w, gate_b))
+        self.runs = cfg.layer_runs()
+        if cfg.loop is not None and (cfg.depth_mix or cfg.out_norm or any(getattr(L.mixer, "kv_from", None) is not None for L in cfg.layers)):
+            raise NotImplementedError("a loop over layers is not combined with depth averages, normed outputs or shared keys and values")
+        self.stream_mix = []                             # per layer: (in, out, mix) of both sublayers, fp32 on the device (no second entry without an MLP)
+        if cfg.streams:
+            if not cfg.sequential or cfg.depth_mix or cfg.out_norm or cfg.bigram is not None or cfg.embed_scale != 1.0:
+                raise NotImplementedError("parallel residual streams are built for plain sequential layers")
+            coef = lambda name, *shape: tensors[name].to(device=self.device, dtype=torch.float32).reshape(shape).contiguous()
+            S = cfg.streams
+            for i, L in enumerate(cfg.layers):
+                self.stream_mix.append([(coef(f"l{i}.hc{q}.in", S), coef(f"l{i}.hc{q}.out", S), coef(f"l{i}.hc{q}.mix", S, S))
+                                        for q in ((1, 2) if L.ff is not None else (1,))])
+        elif any(L.kind == "parallel" and L.mixer.out_norms for L in cfg.layers):
+            raise NotImplementedError("the norms on a parallel mixer's sides are formed where the residual is parallel streams")
         self.has_state = any(L.kind not in ("attention", "latent_attention") for L in cfg.layers)
         self.norm_center = cfg.norm_kind == "layer"
         if cfg.norm_kind not in ("rms", "layer") or (cfg.norm_kind == "layer" and not cfg.out_norm):
@@ -362,23 +442,23 @@ class HybridModel:
 
     # ---- what an engine has to allocate
     def cache_layout(self):
-        """Per layer: ("kv", K page shape, V page shape) | ("kv_from", layer) | ("latent", page shape) | ("state", per-slot shape) |
+        """Per layer run: ("kv", K page shape, V page shape) | ("kv_from", layer) | ("latent", page shape) | ("state", per-slot shape, ...) |
         ("sides", [entries of the two sides of a parallel mixer, each "kv" or "state"])."""
         out = []
-        for L, mixer, *_ in self.layers:
+        for L, mixer, *_ in (self.layers[i] for i in self.runs):
             if L.kind == "parallel":
-                out.append(("sides", [(("kv",) + m.cache_shapes()) if m.cache_kind() == "kv" else ("state", m.state_shape()) for m in (mixer.left, mixer.right)]))
+                out.append(("sides", [(("kv",) + m.cache_shapes()) if m.cache_kind() == "kv" else ("state", *state_shapes(m)) for m in (mixer.left, mixer.right)]))
             elif L.kind == "attention":
                 out.append((("kv",) + mixer.cache_shapes()) if mixer.owns_cache else ("kv_from", L.mixer.kv_from))
             elif L.kind == "latent_attention":
                 out.append(("latent", mixer.cache_shape()))
             else:
-                out.append(("state", mixer.state_shape()))
+                out.append(("state", *state_shapes(mixer)))
         return out
 
     def alloc_cache(self, num_pages: int, num_slots: int):
-        """Cache tensors for `num_pages` pages and `num_slots` state slots: per layer (kcache, vcache) or a state tensor; for a parallel mixer
-        the tuple of its sides' tensors in order."""
+        """Cache tensors for `num_pages` pages and `num_slots` state slots: per layer run (kcache, vcache) or a state tensor (a tuple of them
+        for a mixer with several); for a parallel mixer the tuple of its sides' tensors in order."""
         caches = []
         pages = lambda shape: torch.zeros(num_pages, *shape, dtype=self.dtype, device=self.device)
         slots = lambda shape: torch.zeros(num_slots, *shape, dtype=torch.float32, device=self.device)
@@ -386,7 +466,7 @@ class HybridModel:
             if ent[0] == "sides":
                 flat = []
                 for e in ent[1]:
-                    flat += [pages(e[1]), pages(e[2])] if e[0] == "kv" else [slots(e[1])]
+                    flat += [pages(e[1]), pages(e[2])] if e[0] == "kv" else [slots(sh) for sh in e[1:]]
                 caches.append(tuple(flat))
             elif ent[0] == "kv":
                 caches.append((torch.zeros(num_pages, *ent[1], dtype=self.dtype, device=self.device),
@@ -396,7 +476,8 @@ class HybridModel:
             elif ent[0] == "latent":                   # one row per token serves as key and (its leading channels) as value
                 caches.append((torch.zeros(num_pages, *ent[1], dtype=self.dtype, device=self.device), None))
             else:
-                caches.append(torch.zeros(num_slots, *ent[1], dtype=torch.float32, device=self.device))
+                states = tuple(slots(sh) for sh in ent[1:])
+                caches.append(states if len(states) > 1 else states[0])
         return caches
 
     # ---- one step
@@ -404,6 +485,8 @@ class HybridModel:
         """fp32 logits [len(batch.want), vocab] of the wanted rows; the caches of every row's sequence are advanced.  collect: receives
         the residual stream after every layer (debugging / tests; costs one extra norm launch per layer)."""
         cfg = self.cfg
+        if cfg.streams:
+            return self._forward_streams(batch, caches, collect)
         if cfg.out_norm:
             return self._forward_out_norm(batch, caches, collect)
         if cfg.sequential:
@@ -411,7 +494,8 @@ class HybridModel:
         x = hops.embed(batch.tokens, self.embed)
         a = b = g = None
         shared = self.n_mix
-        for i, ((L, mixer, mlp, n1, n2, gate_w, gate_b), cache) in enumerate(zip(self.layers, caches)):
+        for i, cache in zip(self.runs, caches):
+            L, mixer, mlp, n1, n2, gate_w, gate_b = self.layers[i]
             h1, h2 = hops.residual_norm(x, a, b, cfg.residual_mult, n1, n2, cfg.eps, weight_offset=cfg.norm_offset, gate=g)
             if collect is not None and a is not None:
                 collect.append(x.clone())
@@ -448,19 +532,20 @@ class HybridModel:
         results X_1 .. of all layers and the embedding output X_0 are kept for the step, and the end of layer i replaces the stream by
         sum_j dwa_i[j] X_j, fused with the last residual update and the next norm."""
         cfg, T = self.cfg, batch.tokens.numel()
-        n_layers = len(self.layers)
+        n_layers = len(self.runs)
         stack = torch.empty(n_layers + 1 if cfg.depth_mix else 0, T, cfg.width, dtype=torch.float32, device=self.device)
         bg = cfg.bigram
         x = hops.embed(batch.tokens, self.embed, prev=batch.prev if bg else None, bigram=self.bigram, mul_prev=bg.mul_prev if bg else 0,
                        mul_cur=bg.mul_cur if bg else 0, copy=stack[0] if cfg.depth_mix else None)
-        h1, _ = hops.residual_norm(x, None, None, 1.0, self.layers[0][3], None, cfg.eps, weight_offset=cfg.norm_offset)
-        for i, ((L, mixer, mlp, n1, n2, _gw, _gb), cache) in enumerate(zip(self.layers, caches)):
+        h1, _ = hops.residual_norm(x, None, None, 1.0, self.layers[self.runs[0]][3], None, cfg.eps, weight_offset=cfg.norm_offset)
+        for i, (li, cache) in enumerate(zip(self.runs, caches)):
+            L, mixer, mlp, n1, n2, _gw, _gb = self.layers[li]
             a = mixer.forward(h1, batch, *cache) if isinstance(cache, tuple) else mixer.forward(h1, batch, cache)
             if mlp is not None:
                 h2, _ = hops.residual_norm(x, a, None, 1.0, n2, None, cfg.eps, weight_offset=cfg.norm_offset)
                 a = mlp.forward(h2)
             last = i + 1 == n_layers
-            nw = self.final_norm if last else self.layers[i + 1][3]
+            nw = self.final_norm if last else self.layers[self.runs[i + 1]][3]
             rows = batch.want if last and collect is None else None
             if cfg.depth_mix:
                 h1 = hops.depth_mix_norm(x, a, stack, i + 1, self.depth_coef[i], nw, cfg.eps, weight_offset=cfg.norm_offset, rows=rows)
@@ -493,6 +578,37 @@ class HybridModel:
                 collect.append(x.clone())
         hf = hops.norm_rows(x, batch.want, self.final_norm, cfg.eps, center=self.norm_center)
         return hops.dense_linear(hf, self.head, out_dtype=torch.float32, softcap=cfg.logit_softcap)
+
+
+    def _forward_streams(self, batch: StepBatch, caches, collect: Optional[list]) -> torch.Tensor:
+        """The step of a member whose residual is S parallel streams.  One launch per boundary: the ended sublayer's result (a parallel mixer's normed
+        sides, a mixture's experts) is summed, all streams are mixed and written, the next sublayer's weighted sum of them is read and normed."""
+        cfg, T = self.cfg, batch.tokens.numel()
+        X = torch.empty(T, cfg.streams, cfg.width, dtype=torch.float32, device=self.device)
+        if not self.runs:
+            hf = hops.streams(X, ids=batch.tokens, table=self.embed, w=self.final_norm, eps=cfg.eps).index_select(0, batch.want)
+            return hops.dense_linear(hf, self.head, out_dtype=torch.float32, softcap=cfg.logit_softcap)
+        h = hops.streams(X, ids=batch.tokens, table=self.embed, read=self.stream_mix[self.runs[0]][0][0], w=self.layers[self.runs[0]][3], eps=cfg.eps)
+        for i, (li, cache) in enumerate(zip(self.runs, caches)):
+            L, mixer, mlp, n1, n2, _gw, _gb = self.layers[li]
+            out = mixer.forward(h, batch, *cache) if isinstance(cache, tuple) else mixer.forward(h, batch, cache)
+            y = dict(zip(("a", "ca", "b", "cb"), out)) if isinstance(out, tuple) else {"a": out}
+            if getattr(mixer, "out_norms", None) is not None:
+                y.update(na=mixer.out_norms[0], nb=mixer.out_norms[1], branch_eps=cfg.eps)
+            mixes = self.stream_mix[li]
+            if mlp is not None:
+                h = hops.streams(X, write=mixes[0][1], mix=mixes[0][2], read=mixes[1][0], w=n2, eps=cfg.eps, **y)
+                out = mlp.forward(h, defer=True) if isinstance(mlp, RoutedExperts) else mlp.forward(h)
+                y = {"moe": out} if isinstance(out, hops.MoeSum) else {"a": out}
+            _, write, mix = mixes[-1]
+            last = i + 1 == len(self.runs)
+            nw, read = (self.final_norm, None) if last else (self.layers[self.runs[i + 1]][3], self.stream_mix[self.runs[i + 1]][0][0])
+            h = hops.streams(X, write=write, mix=mix, read=read, w=nw, eps=cfg.eps, rows=batch.want if last and collect is None else None, **y)
+            if collect is not None:
+                collect.append(X.sum(1))
+        if collect is not None:
+            h = hops.streams(X, rows=batch.want, w=self.final_norm, eps=cfg.eps)
+        return hops.dense_linear(h, self.head, out_dtype=torch.float32, softcap=cfg.logit_softcap)
 
 
 def load_hybrid_checkpoint(path: str, dtype: torch.dtype, device, page: int = 64) -> HybridModel:

@@ -9,8 +9,8 @@ import torch
 
 from . import _C
 
-ACT_NONE, ACT_RELU, ACT_SILU, ACT_GELU_TANH, ACT_TANH, ACT_SWIGLU_CLAMP = 0, 1, 2, 3, 4, 5
-ACTIVATIONS = {"none": ACT_NONE, "relu": ACT_RELU, "silu": ACT_SILU, "gelu_tanh": ACT_GELU_TANH, "tanh": ACT_TANH, "swiglu_clamp": ACT_SWIGLU_CLAMP}
+ACT_NONE, ACT_RELU, ACT_SILU, ACT_GELU_TANH, ACT_TANH, ACT_SWIGLU_CLAMP, ACT_RELU2 = 0, 1, 2, 3, 4, 5, 6
+ACTIVATIONS = {"none": ACT_NONE, "relu": ACT_RELU, "silu": ACT_SILU, "gelu_tanh": ACT_GELU_TANH, "tanh": ACT_TANH, "swiglu_clamp": ACT_SWIGLU_CLAMP, "relu2": ACT_RELU2}
 SCAN_HGRN2, SCAN_GLA, SCAN_FIXED, SCAN_FIXED_SILU = 0, 1, 2, 3
 LAYOUTS = {"interleaved": 0, "halves": 1}
 
@@ -219,6 +219,54 @@ class MoeSum:
         self.y, self.place_of, self.wts, self.extra, self.extra_gate = y, place_of, wts, extra, extra_gate
 
 
+def streams(X: torch.Tensor, *, mix: Optional[torch.Tensor] = None, write: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None,
+            a: Optional[torch.Tensor] = None, ca: float = 1.0, na: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None, cb: float = 1.0,
+            nb: Optional[torch.Tensor] = None, branch_eps: float = 0.0, moe: Optional[MoeSum] = None, ids: Optional[torch.Tensor] = None,
+            table: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None, eps: float = 0.0) -> Optional[torch.Tensor]:
+    """The boundary between two sublayers of a model whose residual is S parallel streams X (fp32 [T, S, W], in place):
+        X_t <- sum_s mix[s, t] X_s + write[t] y    (left out without mix),     -> RMS norm of sum_t read[t] X_t under w   (read None: the plain sum)
+    y = ca A + cb B + the mixture sum `moe`, A and B the fp32 [T, W] tensors a and b, RMS-normed over the row under na / nb first when those are given.
+    ids + table: the streams start as the tokens' embedding rows (then there is no y).  rows (int32): only these rows are normed, X is left as it
+    is.  -> [n, W] in w's dtype, None without w."""
+    _dev(X, torch.float32, "streams.X")
+    if X.dim() != 3 or not X.is_contiguous():
+        raise _C.Mi355Error(f"streams: X {tuple(X.shape)} must be contiguous [T, S, W]")
+    T, S, W = X.shape
+    for t, shape, nm in ((mix, (S, S), "mix"), (write, (S,), "write"), (read, (S,), "read"), (a, (T, W), "a"), (b, (T, W), "b")):
+        if t is not None:
+            _dev(t, torch.float32, "streams." + nm)
+            if t.shape != shape or not t.is_contiguous():
+                raise _C.Mi355Error(f"streams.{nm}: {tuple(t.shape)} for {tuple(shape)}")
+    dt = next((t.dtype for t in (w, na, nb, table) if t is not None), torch.float32)
+    for t, n, nm in ((w, W, "w"), (na, W, "na"), (nb, W, "nb")):
+        if t is not None:
+            _dev(t, dt, "streams." + nm)
+            if t.numel() != n or not t.is_contiguous():
+                raise _C.Mi355Error(f"streams.{nm}: {tuple(t.shape)} for width {W}")
+    if moe is not None:
+        _dev(moe.y, torch.float32, "streams.moe.y"); _dev(moe.wts, torch.float32, "streams.moe.wts"); _dev(moe.place_of, torch.int32, "streams.moe.place")
+        if moe.wts.shape[0] != T or moe.y.shape != (moe.wts.numel(), W) or moe.place_of.numel() != moe.wts.numel() or not (moe.y.is_contiguous() and moe.wts.is_contiguous()):
+            raise _C.Mi355Error(f"streams: mixture sum y {tuple(moe.y.shape)} wts {tuple(moe.wts.shape)} against streams {tuple(X.shape)}")
+        if moe.extra is not None:
+            if moe.extra_gate is not None or b is not None:
+                raise _C.Mi355Error("streams: a shared expert joins as the second branch, without a gate")
+            b, cb = moe.extra, 1.0
+    if ids is not None:
+        _dev(ids, torch.int32, "streams.ids"); _dev(table, dt, "streams.table")
+        if ids.numel() != T or table.shape[1] != W or not table.is_contiguous():
+            raise _C.Mi355Error(f"streams: {ids.numel()} ids of a table {tuple(table.shape)} for {T} rows of {W}")
+    if rows is not None:
+        _dev(rows, torch.int32, "streams.rows")
+    n = T if rows is None else rows.numel()
+    h = torch.empty(n, W, dtype=dt, device=X.device) if w is not None else None
+    if n:
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_streams(X.data_ptr(), n, S, W, _p(a), float(ca), _p(na), _p(b), float(cb), _p(nb), float(branch_eps),
+                                                         _p(moe.y) if moe else None, _p(moe.place_of) if moe else None, _p(moe.wts) if moe else None,
+                                                         moe.wts.shape[1] if moe else 0, _p(mix), _p(write), _p(read), _p(ids), _p(table),
+                                                         table.shape[0] if table is not None else 0, _p(rows), _p(w), float(eps), _p(h), act_code(dt), _stream()), "hy_streams")
+    return h
+
+
 def residual_norm(x: torch.Tensor, a: Optional[torch.Tensor], b, mult: float, w1: torch.Tensor,
                   w2: Optional[torch.Tensor], eps: float, *, weight_offset: float = 0.0, rows: Optional[torch.Tensor] = None,
                   gate: Optional[torch.Tensor] = None):
@@ -297,14 +345,15 @@ def _sink(sink: Optional[torch.Tensor], heads: int):
     return _p(sink)
 
 
-def _ogate(gate: Optional[torch.Tensor], T: int, heads: int, name: str):
+def _ogate(gate: Optional[torch.Tensor], T: int, heads: int, vdim: int, name: str):
+    """-> (pointer, row stride, 1 when the gate has a number per value channel instead of one per head)."""
     if gate is None:
-        return None, 0
+        return None, 0, 0
     _dev(gate, torch.float32, name)
     ld = _rows(gate, name)
-    if gate.shape != (T, heads):
-        raise _C.Mi355Error(f"{name}: {tuple(gate.shape)} for {T} rows of {heads} heads")
-    return gate.data_ptr(), ld
+    if gate.shape not in ((T, heads), (T, heads * vdim)):
+        raise _C.Mi355Error(f"{name}: {tuple(gate.shape)} for {T} rows of {heads} heads of {vdim}")
+    return gate.data_ptr(), ld, 1 if gate.shape[1] == heads * vdim and vdim > 1 else 0
 
 
 def attn_rows(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[torch.Tensor], vfreq, pos, seq, block_table, kcache, vcache,
@@ -312,13 +361,13 @@ def attn_rows(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[to
     """Attention of every row over its sequence's pages -> [T, heads * vdim] in the cache dtype.  sink: fp32 [heads] or None; exp(sink[h])
     joins head h's softmax denominator.  Few rows over long block tables (decode steps) are dealt over several blocks per (row, head) whose
     partial sums a second launch merges; the count depends on the rows and the table's width only.  window > 0: a row at position i sees
-    the keys j with 0 <= i - j < window; softcap > 0: cap * tanh(score / cap) on the scaled scores; out_gate fp32 [T, heads] (a column slice is
-    fine): head h of a row is multiplied by the sigmoid of its entry."""
+    the keys j with 0 <= i - j < window; softcap > 0: cap * tanh(score / cap) on the scaled scores; out_gate fp32 [T, heads] or [T, heads * vdim]
+    (a column slice is fine): head h of a row, or every channel of it, is multiplied by the sigmoid of its entry."""
     _dev(q, torch.float32, "attn_rows.q")
     T = q.shape[0]
     out = torch.empty(T, heads * vdim, dtype=kcache.dtype, device=q.device)
     splits, parts = 1, None
-    gp, ldg = _ogate(out_gate, T, heads, "attn_rows.out_gate")
+    gp, ldg, gch = _ogate(out_gate, T, heads, vdim, "attn_rows.out_gate")
     if chunk == 0 and T * heads <= 2048:                   # sixteen waves per block: one 64-key tile per wave and block where the chip has room
         tiles = (block_table.shape[1] * geom[7] + 63) // 64
         if window > 0:
@@ -327,9 +376,9 @@ def attn_rows(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[to
         if splits > 1:
             parts = torch.empty(T * heads * splits * (vdim + 2), dtype=torch.float32, device=q.device)
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_rows_ex(q.data_ptr(), _rows(q, "attn_rows.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_rows_ex2(q.data_ptr(), _rows(q, "attn_rows.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
                                                               pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), T, kcache.data_ptr(), vcache.data_ptr(),
-                                                              out.data_ptr(), splits, _p(parts), int(window), float(softcap), gp, ldg, act_code(kcache.dtype),
+                                                              out.data_ptr(), splits, _p(parts), int(window), float(softcap), gp, ldg, gch, act_code(kcache.dtype),
                                                               _stream()), "hy_attn_rows")
     return out
 
@@ -346,12 +395,12 @@ def attn_tiles(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[t
     _dev(q, torch.float32, "attn_tiles.q"); _dev(tile_row0, torch.int32, "attn_tiles.tile_row0"); _dev(tile_n, torch.int32, "attn_tiles.tile_n")
     T = q.shape[0]
     out = torch.empty(T, heads * vdim, dtype=kcache.dtype, device=q.device)
-    gp, ldg = _ogate(out_gate, T, heads, "attn_tiles.out_gate")
+    gp, ldg, gch = _ogate(out_gate, T, heads, vdim, "attn_tiles.out_gate")
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_tiles_ex(q.data_ptr(), _rows(q, "attn_tiles.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_tiles_ex2(q.data_ptr(), _rows(q, "attn_tiles.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
                                                                pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), tile_row0.data_ptr(), tile_n.data_ptr(),
                                                                tile_row0.numel(), kcache.data_ptr(), vcache.data_ptr(), out.data_ptr(), int(window),
-                                                               float(softcap), gp, ldg, act_code(kcache.dtype), _stream()), "hy_attn_tiles")
+                                                               float(softcap), gp, ldg, gch, act_code(kcache.dtype), _stream()), "hy_attn_tiles")
     return out
 
 
@@ -416,8 +465,19 @@ def scan(mode: int, proj: torch.Tensor, qo: int, ko: int, vo: int, z: Optional[t
     if not fixed or not state.is_contiguous() or state.shape[1:] != (heads, dim, vdim):
         raise _C.Mi355Error(f"scan: the chunked form takes a constant decay per head and a contiguous state [slots, {heads}, {dim}, {vdim}]")
     _dev(lower, torch.float32, "scan.decay")
+    plan = _chunk_plan(row_start, T, nseq, heads * dim * vdim * 4, plans)
+    cstate = torch.empty(plan.max_chunks, heads, dim, vdim, dtype=torch.float32, device=proj.device)
+    run(mode, plan.cs, plan.ids, plan.zeros, plan.max_chunks, cstate)                       # 1: every chunk from a zero state
+    _C.check_hybrid(lib.mi355_hy_chunk_prefix(plan.cs.data_ptr(), plan.sc.data_ptr(), slot.data_ptr(), first_pos.data_ptr(), nseq, lower.data_ptr(), heads,
+                                              dim * vdim, cstate.data_ptr(), state.data_ptr(), _stream()), "hy_chunk_prefix")        # 2: states at the chunks' starts
+    run(mode + 4, plan.cs, plan.ids, plan.ones, plan.max_chunks, cstate)                    # 3: their share of the outputs
+    return out
+
+
+def _chunk_plan(row_start, T: int, nseq: int, per_chunk_bytes: int, plans: Optional[dict]) -> ChunkPlan:
+    """The step's plan with chunks of SCAN_CHUNK rows, or of more when the chunk states would not fit the scratch limit."""
     C = SCAN_CHUNK
-    while (T // C + nseq + 1) * heads * dim * vdim * 4 > SCAN_CHUNK_BYTES and C < T:
+    while (T // C + nseq + 1) * per_chunk_bytes > SCAN_CHUNK_BYTES and C < T:
         C *= 2
     key = (row_start.data_ptr(), T, nseq, C)
     plan = plans.get(key) if plans is not None else None
@@ -426,11 +486,103 @@ def scan(mode: int, proj: torch.Tensor, qo: int, ko: int, vo: int, z: Optional[t
         if plans is not None:
             plans.clear()
             plans[key] = plan
-    cstate = torch.empty(plan.max_chunks, heads, dim, vdim, dtype=torch.float32, device=proj.device)
-    run(mode, plan.cs, plan.ids, plan.zeros, plan.max_chunks, cstate)                       # 1: every chunk from a zero state
-    _C.check_hybrid(lib.mi355_hy_chunk_prefix(plan.cs.data_ptr(), plan.sc.data_ptr(), slot.data_ptr(), first_pos.data_ptr(), nseq, lower.data_ptr(), heads,
-                                              dim * vdim, cstate.data_ptr(), state.data_ptr(), _stream()), "hy_chunk_prefix")        # 2: states at the chunks' starts
-    run(mode + 4, plan.cs, plan.ids, plan.ones, plan.max_chunks, cstate)                    # 3: their share of the outputs
+    return plan
+
+
+def memory_scan(proj: torch.Tensor, qo: int, ko: int, vo: int, io: int, fo: int, cap: float, qscale: float, den_eps: float, heads: int, dim: int, vdim: int,
+                row_start, slot, first_pos, state: torch.Tensor, mstate: torch.Tensor, *, plans: Optional[dict] = None, chunked: Optional[bool] = None,
+                max_rows: int = 0):
+    """Matrix memory under exponential gates over the rows of every sequence -> (o fp32 [T, heads * vdim], den fp32 [T, heads]): per head, with log gates
+    i = cap tanh(proj[io + h] / cap), f = log sigmoid(cap tanh(proj[fo + h] / cap)) and m_t = max(f + m_(t-1), i),
+        S <- e^(f + m_(t-1) - m_t) S + e^(i - m_t) k v^T,  n likewise with k alone,  o = S^T (qscale q),  den = max(|n . (qscale q)|, e^(-m_t)) + den_eps.
+    The quotient o / den is left to the norm behind it.  state fp32 [slots, heads, dim * vdim + dim] holds S and n, mstate [slots, heads, ceil(vdim / 64)]
+    the running maximum.  Long prompt portions run in chunks walked side by side, as in `scan` (plans, chunked, max_rows as there)."""
+    _dev(proj, torch.float32, "memory_scan.proj"); _dev(state, torch.float32, "memory_scan.state"); _dev(mstate, torch.float32, "memory_scan.mstate")
+    T, ld, nz = proj.shape[0], _rows(proj, "memory_scan.proj"), (vdim + 63) // 64
+    if (max(qo, ko) + heads * dim > proj.shape[1] or vo + heads * vdim > proj.shape[1] or max(io, fo) + heads > proj.shape[1]
+            or state.shape[1:] != (heads, dim * vdim + dim) or mstate.shape[1:] != (heads, nz) or not state.is_contiguous() or not mstate.is_contiguous()):
+        raise _C.Mi355Error(f"memory_scan: proj {tuple(proj.shape)} state {tuple(state.shape)} / {tuple(mstate.shape)} for {heads} heads of {dim} x {vdim}")
+    out = torch.empty(T, heads * vdim, dtype=torch.float32, device=proj.device)
+    den = torch.empty(T, heads, dtype=torch.float32, device=proj.device)
+    nseq = slot.numel()
+    if not (T and nseq):
+        return out, den
+    lib = _C.hybrid_lib()
+
+    def run(which, rs, sl, fp, n, st, gates, cdecay):
+        _C.check_hybrid(lib.mi355_hy_memory_scan(which, proj.data_ptr(), ld, qo, ko, vo, io, fo, float(cap), float(qscale), float(den_eps), heads, dim, vdim,
+                                                 rs.data_ptr(), sl.data_ptr(), fp.data_ptr(), n, st.data_ptr(), mstate.data_ptr(), _p(gates), _p(cdecay),
+                                                 den.data_ptr(), out.data_ptr(), _stream()), "hy_memory_scan")
+
+    if chunked is None:
+        chunked = scan_prefers_chunks(T, nseq, max_rows, heads, vdim, SCAN_CHUNK)
+    if not chunked:
+        run(0, row_start, slot, first_pos, nseq, state, None, None)
+        return out, den
+    per_head = dim * vdim + dim
+    plan = _chunk_plan(row_start, T, nseq, heads * per_head * 4, plans)
+    gates = torch.empty(T, heads, 3, dtype=torch.float32, device=proj.device)
+    cstate = torch.empty(plan.max_chunks, heads, per_head, dtype=torch.float32, device=proj.device)
+    cdecay = torch.empty(plan.max_chunks, heads, dtype=torch.float32, device=proj.device)
+    _C.check_hybrid(lib.mi355_hy_memory_gates(proj.data_ptr(), ld, io, fo, float(cap), heads, row_start.data_ptr(), slot.data_ptr(), first_pos.data_ptr(), nseq,
+                                              mstate.data_ptr(), nz, gates.data_ptr(), _stream()), "hy_memory_gates")
+    run(1, plan.cs, plan.ids, plan.zeros, plan.max_chunks, cstate, gates, cdecay)
+    _C.check_hybrid(lib.mi355_hy_chunk_prefix_ex(plan.cs.data_ptr(), plan.sc.data_ptr(), slot.data_ptr(), first_pos.data_ptr(), nseq, None, cdecay.data_ptr(), heads,
+                                                 per_head, cstate.data_ptr(), state.data_ptr(), _stream()), "hy_chunk_prefix")
+    run(2, plan.cs, plan.ids, plan.ones, plan.max_chunks, cstate, gates, None)
+    return out, den
+
+
+def short_conv(proj: torch.Tensor, channels: int, w: torch.Tensor, hist: Optional[torch.Tensor], seq, row_start, slot, first_pos, *, unit_heads: int = 0,
+               query_heads: int = 0, dim: int = 0, qscale: float = 1.0, unit_eps: float = 1e-6, low: Optional[tuple] = None):
+    """Causal convolutions over time, one per channel of proj[:, :channels] under w [channels, taps] (last tap: the current token), then silu -> fp32
+    [T, channels].  The first unit_heads heads of `dim` channels are brought to unit length, the first query_heads of them times qscale.  hist fp32
+    [slots, taps - 1, channels]: the raw rows before the step (None for one tap); they are only read here and moved on by the recurrence's kernel.
+    low = (column, count): these columns of proj come back rounded to w's dtype as a second tensor."""
+    _dev(proj, torch.float32, "short_conv.proj")
+    T, taps = proj.shape[0], w.shape[1]
+    if w.shape[0] != channels or not w.is_contiguous() or proj.shape[1] < channels or (taps > 1 and (hist is None or hist.shape[1:] != (taps - 1, channels) or not hist.is_contiguous())):
+        raise _C.Mi355Error(f"short_conv: proj {tuple(proj.shape)} weights {tuple(w.shape)} history {None if hist is None else tuple(hist.shape)} for {channels} channels")
+    if hist is not None:
+        _dev(hist, torch.float32, "short_conv.hist")
+    out = torch.empty(T, channels, dtype=torch.float32, device=proj.device)
+    lo, R = low if low is not None else (0, 0)
+    lowt = torch.empty(T, R, dtype=w.dtype, device=proj.device) if low is not None else None
+    if T:
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_short_conv(proj.data_ptr(), _rows(proj, "short_conv.proj"), T, channels, taps, w.data_ptr(), unit_heads, query_heads, dim,
+                                                            float(qscale), float(unit_eps), _p(hist), seq.data_ptr(), row_start.data_ptr(), slot.data_ptr(),
+                                                            first_pos.data_ptr(), out.data_ptr(), lo, R, _p(lowt), act_code(w.dtype), _stream()), "hy_short_conv")
+    return out, lowt
+
+
+def channel_delta_scan(x: torch.Tensor, ro: int, ko: int, vo: int, z: torch.Tensor, zbias: torch.Tensor, rate: torch.Tensor, steps: torch.Tensor, heads: int,
+                       kv_heads: int, dim: int, vdim: int, row_start, slot, first_pos, state: torch.Tensor, *, raw: Optional[torch.Tensor] = None,
+                       hist: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Delta rule with a decay per key channel over the rows of every sequence: S <- diag(g) S, u = beta (v - S^T k), S <- S + k u^T, o = S^T r with
+    g = exp(-rate[h] softplus(z + zbias)) (z fp32 [T, heads * dim], zbias fp32 [heads * dim], rate fp32 [heads]) and beta = sigmoid(steps) (fp32 [T, heads], a
+    column slice is fine).  r and k (kv_heads heads of dim, head h reads h // (heads / kv_heads)) and v (heads of vdim) are columns ro, ko, vo of x.
+    Continues and leaves the state [slots, heads, dim, vdim]; with hist (the short convolution's rows, [slots, taps - 1, C]) and raw (its inputs, columns
+    0 .. C - 1) the slots' rows are moved on as well.  -> fp32 [T, heads * vdim]."""
+    for t, nm in ((x, "x"), (z, "z"), (zbias, "zbias"), (rate, "rate"), (steps, "steps"), (state, "state")):
+        _dev(t, torch.float32, "channel_delta_scan." + nm)
+    T = x.shape[0]
+    if (max(ro, ko) + kv_heads * dim > x.shape[1] or vo + heads * vdim > x.shape[1] or z.shape != (T, heads * dim) or zbias.numel() != heads * dim or rate.numel() != heads
+            or steps.shape != (T, heads) or state.shape[1:] != (heads, dim, vdim) or not state.is_contiguous()):
+        raise _C.Mi355Error(f"channel_delta_scan: x {tuple(x.shape)} z {tuple(z.shape)} state {tuple(state.shape)} for {heads} heads ({kv_heads} key heads) of {dim} x {vdim}")
+    taps = C = ldr = 0
+    if hist is not None:
+        _dev(hist, torch.float32, "channel_delta_scan.hist"); _dev(raw, torch.float32, "channel_delta_scan.raw")
+        taps, C, ldr = hist.shape[1] + 1, hist.shape[2], _rows(raw, "channel_delta_scan.raw")
+        if raw.shape[0] != T or raw.shape[1] < C or not hist.is_contiguous():
+            raise _C.Mi355Error(f"channel_delta_scan: raw {tuple(raw.shape)} for a history {tuple(hist.shape)}")
+    out = torch.empty(T, heads * vdim, dtype=torch.float32, device=x.device)
+    nseq = slot.numel()
+    if T and nseq:
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_channel_delta_scan(x.data_ptr(), _rows(x, "channel_delta_scan.x"), ro, ko, vo, z.data_ptr(),
+                                                                    _rows(z, "channel_delta_scan.z"), zbias.data_ptr(), rate.data_ptr(), steps.data_ptr(),
+                                                                    _rows(steps, "channel_delta_scan.steps"), heads, kv_heads, dim, vdim, row_start.data_ptr(),
+                                                                    slot.data_ptr(), first_pos.data_ptr(), nseq, state.data_ptr(), out.data_ptr(), _p(raw), ldr, C,
+                                                                    taps, _p(hist), _stream()), "hy_channel_delta_scan")
     return out
 
 
@@ -456,9 +608,10 @@ def delta_scan(proj: torch.Tensor, ro: int, ko: int, vo: int, ao: int, z: torch.
 
 
 def head_norm(o: torch.Tensor, heads: int, vdim: int, w: Optional[torch.Tensor], eps: float, gate: Optional[torch.Tensor] = None, goff: int = 0,
-              out_dtype: Optional[torch.dtype] = None, gate_act: str = "silu") -> torch.Tensor:
+              out_dtype: Optional[torch.dtype] = None, gate_act: str = "silu", den: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per-head RMS norm of o (fp32 [T, heads * vdim]) under the weight w ([vdim] shared by the heads, or [heads * vdim]; None: unit RMS only,
-    output in `out_dtype`), times gate_act(gate[:, goff:]) ("silu" or "sigmoid") when a gate is given."""
+    output in `out_dtype`), times gate_act(gate[:, goff:]) ("silu" or "sigmoid") when a gate is given.  den (fp32 [T, heads]): every head is divided
+    by its entry before the norm."""
     _dev(o, torch.float32, "head_norm.o")
     T = o.shape[0]
     dt = w.dtype if w is not None else out_dtype
@@ -471,9 +624,13 @@ def head_norm(o: torch.Tensor, heads: int, vdim: int, w: Optional[torch.Tensor],
     if gate_act not in ("silu", "sigmoid"):
         raise _C.Mi355Error(f"head_norm: gate activation {gate_act!r}")
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_head_norm_ex(o.data_ptr(), T, heads, vdim, _p(w), float(eps), _p(gate),
+        if den is not None:
+            _dev(den, torch.float32, "head_norm.den")
+            if den.shape != (T, heads) or not den.is_contiguous():
+                raise _C.Mi355Error(f"head_norm: denominators {tuple(den.shape)} for {T} rows of {heads} heads")
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_head_norm_ex2(o.data_ptr(), T, heads, vdim, _p(w), float(eps), _p(gate),
                                                               0 if gate is None else _rows(gate, "head_norm.gate"), goff, out.data_ptr(), per_head,
-                                                              1 if gate_act == "sigmoid" else 0, act_code(dt), _stream()), "hy_head_norm")
+                                                              1 if gate_act == "sigmoid" else 0, _p(den), act_code(dt), _stream()), "hy_head_norm")
     return out
 
 
@@ -575,8 +732,9 @@ def polynorm(z: torch.Tensor, coef, eps: float, dtype: torch.dtype) -> torch.Ten
     return out
 
 
-def moe_route(z: torch.Tensor, groups: int, keep: int, top: int, *, sigmoid: bool = False, group_top: int = 1, scale: float = 1.0):
-    """Router logits fp32 [T, E] -> (expert ids int32 [T, top], weights fp32 [T, top]): softmax scores (sigmoid: a sigmoid of every logit), only
+def moe_route(z: torch.Tensor, groups: int, keep: int, top: int, *, sigmoid: bool = False, chosen: bool = False, group_top: int = 1, scale: float = 1.0):
+    """Router logits fp32 [T, E] -> (expert ids int32 [T, top], weights fp32 [T, top]): softmax scores (sigmoid: a sigmoid of every logit; chosen: softmax
+    over the chosen logits alone), only
     experts of the `keep` best of `groups` runs of neighbouring experts (a run scores as its best member, or with group_top = 2 as the sum of its
     two best) are eligible, the `top` best eligible are chosen; their weights are score * scale."""
     _dev(z, torch.float32, "moe_route.z")
@@ -585,7 +743,7 @@ def moe_route(z: torch.Tensor, groups: int, keep: int, top: int, *, sigmoid: boo
     wts = torch.empty(T, top, dtype=torch.float32, device=z.device)
     if T:
         _C.check_hybrid(_C.hybrid_lib().mi355_hy_moe_route_ex(z.data_ptr(), _rows(z, "moe_route.z"), T, E, groups, keep, top, ids.data_ptr(), wts.data_ptr(),
-                                                              1 if sigmoid else 0, int(group_top), float(scale), _stream()), "hy_moe_route")
+                                                              2 if chosen else 1 if sigmoid else 0, int(group_top), float(scale), _stream()), "hy_moe_route")
     return ids, wts
 
 
@@ -605,14 +763,14 @@ def moe_align(ids: torch.Tensor, experts: int):
     return offs, src, place, tiles
 
 
-def moe_route_sorted(z: torch.Tensor, experts: int, groups: int, keep: int, top: int, *, sigmoid: bool = False, group_top: int = 1, scale: float = 1.0):
+def moe_route_sorted(z: torch.Tensor, experts: int, groups: int, keep: int, top: int, *, sigmoid: bool = False, chosen: bool = False, group_top: int = 1, scale: float = 1.0):
     """moe_route followed by moe_align -> (ids, wts, offs, src_row, place_of, tiles); a few tokens (a decode step) take one launch for both."""
     _dev(z, torch.float32, "moe_route_sorted.z")
     T = z.shape[0]
     if z.shape[1] != experts:
         raise _C.Mi355Error(f"moe_route_sorted: logits {tuple(z.shape)} for {experts} experts")
     if not 0 < T <= 64 or 16 * (experts + groups) * 4 + experts * 8 > 48 * 1024:
-        ids, wts = moe_route(z, groups, keep, top, sigmoid=sigmoid, group_top=group_top, scale=scale)
+        ids, wts = moe_route(z, groups, keep, top, sigmoid=sigmoid, chosen=chosen, group_top=group_top, scale=scale)
         return (ids, wts) + moe_align(ids, experts)
     dev = z.device
     ids, wts = torch.empty(T, top, dtype=torch.int32, device=dev), torch.empty(T, top, dtype=torch.float32, device=dev)
@@ -620,7 +778,7 @@ def moe_route_sorted(z: torch.Tensor, experts: int, groups: int, keep: int, top:
     tiles = torch.empty(1 + 2 * (T * top // 64 + experts), dtype=torch.int32, device=dev)
     _C.check_hybrid(_C.hybrid_lib().mi355_hy_moe_route_align_ex(z.data_ptr(), _rows(z, "moe_route_sorted.z"), T, experts, groups, keep, top, ids.data_ptr(),
                                                                 wts.data_ptr(), offs.data_ptr(), src.data_ptr(), place.data_ptr(), tiles.data_ptr(),
-                                                                1 if sigmoid else 0, int(group_top), float(scale), _stream()), "hy_moe_route_align")
+                                                                2 if chosen else 1 if sigmoid else 0, int(group_top), float(scale), _stream()), "hy_moe_route_align")
     return ids, wts, offs, src, place, tiles
 
 

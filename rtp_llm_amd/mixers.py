@@ -21,10 +21,14 @@
     attention over the cached rows.  Rotary with optional YaRN frequency scaling, a learned per-head softmax sink, a sigmoid output gate.
   * ``Retention`` -- the same recurrence with one constant decay per head, rotated q and k, unit-RMS heads and a silu output gate.
   * ``LightningAttention`` -- that recurrence with silu on q, k and v, one RMS norm over all heads together and a sigmoid output gate.
-  * ``ParallelMixer`` -- two of the mixers side by side on one input, their outputs added with a constant each.
+  * ``ChannelDelta`` -- the gated delta rule with a decay per key channel, S <- diag(g) S, S <- S + beta k (v - S^T k)^T, o = S^T q, on unit queries and
+    keys that (like the values) have passed a short causal convolution; low-rank decay and output gate, unit-RMS heads.
+  * ``MatrixMemory`` -- S_t = e^f S_(t-1) + e^i k v^T, n_t likewise with k alone, o = S^T q / max(|n . q|, 1), with the exponentials kept in range by a running
+    maximum (carried with the state); unit-RMS heads under a weight per channel and a sigmoid output gate.
+  * ``ParallelMixer`` -- two of the mixers side by side on one input, their outputs added with a constant each (optionally RMS-normed first).
   * ``GatedMLP``, ``PolyNormMLP``, ``RoutedExperts`` -- feed-forward branches: gated dense, dense with the PolyNorm activation, and a
-    mixture of gated experts (softmax or sigmoid router, group-limited top-k, optional shared expert with an optional gate of its own) over
-    one grouped linear per projection.  The gated activations include the clamped form min(g, L) sigmoid(1.702 min(g, L)) (clamp(u) + 1).
+    mixture of gated or plain experts (softmax or sigmoid router, softmax over the chosen logits alone, group-limited top-k, optional shared expert
+    with an optional gate of its own) over one grouped linear per projection.  The gated activations include the clamped form min(g, L) sigmoid(1.702 min(g, L)) (clamp(u) + 1).
 
 All take the normed activations of a ragged batch (``StepBatch``) and return the fp32 branch output [T, width]."""
 import math
@@ -101,7 +105,8 @@ class AttentionSpec:
     qk_norm: bool = False                # queries and keys are RMS-normed per head under weights [dim] shared by the heads, before the rotation
     bias: bool = False                   # the q, k, v projections have biases
     out_bias: bool = False               # the output projection has a bias
-    out_gate: bool = False               # head h's output is multiplied by sigmoid(W_g x)_h, one number per head
+    out_gate: bool = False               # head h's output is multiplied by sigmoid(W_g x)_h, one number per head ...
+    gate_channels: bool = False          # ... with out_gate: one number per head and value channel
     learned_sink: bool = False           # with sink: head h's sink logit is the checkpoint's `sink`[h] instead of 0
     qk_norm_whole: bool = False          # with qk_norm: ONE RMS norm over all query heads (and one over all key heads) under weights [heads * dim]
 
@@ -174,7 +179,7 @@ def rotary_steps(n_pairs: int, span: int, base: float, device) -> torch.Tensor:
 
 class PagedChunkAttention:
     """weights: q [H dim, W], k [G dim, W], v [G vdim, W] (absent with kv_from), o [W, H vdim]; by option q.b / k.b / v.b / o.b, q.norm / k.norm [dim]
-    (or [H dim] / [G dim] when the norm runs over all heads at once), g [H, W], sink [H].  Every projection of the input (q | k | v | gate) is one
+    (or [H dim] / [G dim] when the norm runs over all heads at once), g [H, W] (or [H vdim, W]), sink [H].  Every projection of the input (q | k | v | gate) is one
     linear."""
 
     def __init__(self, spec: AttentionSpec, weights: Dict[str, torch.Tensor], eps: float, page: int, device):
@@ -185,12 +190,15 @@ class PagedChunkAttention:
         if s.window and s.chunk:
             raise ValueError("attention: a sliding window and a block mask exclude each other")
         self.owns_cache = s.kv_from is None
+        self.n_gate = 0 if not s.out_gate else s.heads * (s.vdim if s.gate_channels else 1)
+        if s.out_gate and weights["g"].shape[0] != self.n_gate:
+            raise ValueError(f"attention: output gate {tuple(weights['g'].shape)} for {s.heads} heads of {s.vdim}")
         names = ["q"] + (["k", "v"] if self.owns_cache else [])
         parts = [weights[n] for n in names] + ([weights["g"]] if s.out_gate else [])
         self.w_in = torch.cat(parts, 0).contiguous()
         self.b_in = None
         if s.bias:
-            zero = [torch.zeros(s.heads, dtype=self.w_in.dtype, device=self.w_in.device)] if s.out_gate else []
+            zero = [torch.zeros(weights["g"].shape[0], dtype=self.w_in.dtype, device=self.w_in.device)] if s.out_gate else []
             self.b_in = torch.cat([weights[n + ".b"] for n in names] + zero, 0).contiguous()
         self.w_o = weights["o"].contiguous()
         self.b_o = weights["o.b"].contiguous() if s.out_bias else None
@@ -242,7 +250,7 @@ class PagedChunkAttention:
                        kcache if write else None, vcache if write else None, q_norm=self.q_norm, k_norm=self.k_norm, mag=self.mag, q_temp=s.q_temp,
                        cache_dtype=kcache.dtype, norm_whole=s.qk_norm_whole)
         T = qkv.shape[0]
-        extra = dict(window=s.window, softcap=s.softcap, out_gate=qkv[:, self.goff:self.goff + s.heads] if s.out_gate else None)
+        extra = dict(window=s.window, softcap=s.softcap, out_gate=qkv[:, self.goff:self.goff + self.n_gate] if s.out_gate else None)
         # prompt portions (tiles mostly full) go to the matrix-core kernel, decode rows to the one that spreads a row's keys over four waves
         if (self.use_tiles and batch.tile_row0 is not None and batch.tile_row0.numel() * 4 <= T
                 and hops.attn_tiles_supported(kcache.dtype, s.dim, s.vdim, self.vfreq is not None, hops.LAYOUTS[s.value_layout])):
@@ -497,14 +505,140 @@ class LightningAttention:
         return hops.dense_linear(o, self.w_o, out_dtype=torch.float32) if out_proj else o
 
 
+@dataclass
+class ChannelDeltaSpec:
+    heads: int
+    kv_heads: int                        # query / key heads; head h reads h // (heads / kv_heads)
+    dim: int
+    vdim: int
+    conv: int                            # taps of the short convolutions
+    unit_eps: float = 1e-6               # q, k: x / sqrt(sum x^2 + unit_eps)
+
+
+class ChannelDelta:
+    """weights: q, k [G dim, W], v [H vdim, W], q.conv / k.conv / v.conv [channels, taps], b [H, W], A_log [H], a1 [Ra, W], a2 [H dim, Ra], dt_bias [H dim],
+    g1 [Rg, W], g2 [H vdim, Rg], norm [vdim], o [W, H vdim].  One linear gives q | k | v | a1 | g1 | b in fp32; one launch runs the convolutions with
+    silu, the unit lengths and the rounding of a1 | g1; ONE grouped linear forms both low-rank products (each padded to the larger of the two); the scan
+    takes decay and step size from their pre-activations.  State per slot: S (fp32) and the convolutions' last taps - 1 raw rows (fp32)."""
+
+    def __init__(self, spec: ChannelDeltaSpec, weights: Dict[str, torch.Tensor], eps: float, device):
+        s = self.spec = spec
+        self.eps = eps
+        if s.heads % s.kv_heads or s.conv < 1:
+            raise ValueError(f"channel delta: {s.heads} heads over {s.kv_heads} key heads, {s.conv} taps")
+        gd, hd, hv = s.kv_heads * s.dim, s.heads * s.dim, s.heads * s.vdim
+        for n, rows in (("q", gd), ("k", gd), ("v", hv), ("b", s.heads), ("a2", hd), ("g2", hv)):
+            if weights[n].shape[0] != rows:
+                raise ValueError(f"channel delta: weight {n} {tuple(weights[n].shape)} for {s.heads} heads ({s.kv_heads} key heads) of {s.dim} x {s.vdim}")
+        for n, rows in (("q.conv", gd), ("k.conv", gd), ("v.conv", hv)):
+            if weights[n].numel() != rows * s.conv:
+                raise ValueError(f"channel delta: {n} {tuple(weights[n].shape)} for {rows} channels of {s.conv} taps")
+        self.channels = 2 * gd + hv
+        self.w_conv = torch.cat([weights[n].reshape(-1, s.conv) for n in ("q.conv", "k.conv", "v.conv")], 0).contiguous()
+        dt = weights["q"].dtype
+        zeros = lambda *sh: torch.zeros(*sh, dtype=dt, device=weights["q"].device)
+        # the low-rank pairs as two groups of one linear: ranks padded to R (a multiple of 8), outputs to N
+        ra, rg = weights["a1"].shape[0], weights["g1"].shape[0]
+        self.R, self.N = -(-max(ra, rg) // 8) * 8, max(hd, hv)
+        W = weights["q"].shape[1]
+        pad_rows = lambda t, n: torch.cat([t, zeros(n - t.shape[0], t.shape[1])], 0)
+        pad_cols = lambda t, n: torch.cat([t, zeros(t.shape[0], n - t.shape[1])], 1)
+        self.lo = -(-self.channels // 4) * 4
+        self.bo = self.lo + 2 * self.R
+        self.w_in = torch.cat([weights["q"], weights["k"], weights["v"], zeros(self.lo - self.channels, W), pad_rows(weights["a1"], self.R),
+                               pad_rows(weights["g1"], self.R), weights["b"]], 0).contiguous()
+        self.b_in = None
+        self.w_low = torch.stack([pad_rows(pad_cols(weights["a2"], self.R), self.N), pad_rows(pad_cols(weights["g2"], self.R), self.N)]).contiguous()
+        self.rate = torch.exp(weights["A_log"].reshape(-1).to(torch.float32)).contiguous()
+        self.zbias = weights["dt_bias"].reshape(-1).to(torch.float32).contiguous()
+        if self.rate.numel() != s.heads or self.zbias.numel() != hd:
+            raise ValueError(f"channel delta: A_log {self.rate.numel()} / dt_bias {self.zbias.numel()} for {s.heads} heads of {s.dim}")
+        self.norm, self.w_o = weights["norm"].contiguous(), weights["o"].contiguous()
+
+    def cache_kind(self):
+        return "state"
+
+    def state_shapes(self):
+        s = self.spec
+        return [(s.heads, s.dim, s.vdim), (s.conv - 1, self.channels)]
+
+    def forward(self, h: torch.Tensor, batch: StepBatch, state: torch.Tensor, hist: torch.Tensor, proj: Optional[torch.Tensor] = None, out_proj: bool = True) -> torch.Tensor:
+        """proj: h w_in^T in fp32 when the caller has computed it.  out_proj False: the normed, gated heads [T, H vdim] come back unprojected."""
+        s = self.spec
+        gd, hd, hv = s.kv_heads * s.dim, s.heads * s.dim, s.heads * s.vdim
+        if proj is None:
+            proj = hops.dense_linear(h, self.w_in, out_dtype=torch.float32)
+        x, low = hops.short_conv(proj, self.channels, self.w_conv, hist, batch.seq, batch.row_start, batch.slot, batch.first_pos, unit_heads=2 * s.kv_heads,
+                                 query_heads=s.kv_heads, dim=s.dim, qscale=s.dim ** -0.5, unit_eps=s.unit_eps, low=(self.lo, 2 * self.R))
+        zg = hops.dense_grouped(low, self.w_low, x_step=self.R, y_step=self.N, out_dtype=torch.float32)
+        o = hops.channel_delta_scan(x, 0, gd, 2 * gd, zg[:, :hd], self.zbias, self.rate, proj[:, self.bo:self.bo + s.heads], s.heads, s.kv_heads, s.dim, s.vdim,
+                                    batch.row_start, batch.slot, batch.first_pos, state, raw=proj, hist=hist)
+        o = hops.head_norm(o, s.heads, s.vdim, self.norm, self.eps, zg, self.N, gate_act="sigmoid")
+        return hops.dense_linear(o, self.w_o, out_dtype=torch.float32) if out_proj else o
+
+
+@dataclass
+class MatrixMemorySpec:
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float                      # both gate pre-activations pass cap tanh(z / cap)
+    den_eps: float = 1e-6                # added to the denominator
+
+
+class MatrixMemory:
+    """weights: q, k [H dim, W], v, g [H vdim, W], i, f [H, W], i.b, f.b [H], norm [H vdim], o [W, H vdim].  One linear gives q | k | v | g | i | f (with the gates'
+    biases) in fp32; the scan forms gates, states and denominators, the norm behind it divides, brings every head to unit RMS, multiplies by norm and
+    by sigmoid(g).  State per slot: S with n behind it, and the running maximum (a copy per block of value columns)."""
+
+    def __init__(self, spec: MatrixMemorySpec, weights: Dict[str, torch.Tensor], eps: float, device):
+        s = self.spec = spec
+        self.eps = eps
+        hd, hv = s.heads * s.dim, s.heads * s.vdim
+        for n, rows in (("q", hd), ("k", hd), ("v", hv), ("g", hv), ("i", s.heads), ("f", s.heads)):
+            if weights[n].shape[0] != rows:
+                raise ValueError(f"matrix memory: weight {n} {tuple(weights[n].shape)} for {s.heads} heads of {s.dim} x {s.vdim}")
+        self.w_in = torch.cat([weights[n] for n in ("q", "k", "v", "g", "i", "f")], 0).contiguous()
+        self.b_in = torch.cat([torch.zeros(2 * hd + 2 * hv, dtype=self.w_in.dtype, device=self.w_in.device), weights["i.b"].reshape(-1), weights["f.b"].reshape(-1)]).contiguous()
+        self.qo, self.ko, self.vo, self.go = 0, hd, 2 * hd, 2 * hd + hv
+        self.io, self.fo = 2 * hd + 2 * hv, 2 * hd + 2 * hv + s.heads
+        self.norm, self.w_o = weights["norm"].contiguous(), weights["o"].contiguous()
+        if self.norm.numel() != hv:
+            raise ValueError(f"matrix memory: norm weight of {self.norm.numel()} channels for {hv}")
+
+    def cache_kind(self):
+        return "state"
+
+    def state_shapes(self):
+        s = self.spec
+        return [(s.heads, s.dim * s.vdim + s.dim), (s.heads, (s.vdim + 63) // 64)]
+
+    def forward(self, h: torch.Tensor, batch: StepBatch, state: torch.Tensor, mstate: torch.Tensor, proj: Optional[torch.Tensor] = None, out_proj: bool = True) -> torch.Tensor:
+        """proj: h w_in^T + b_in in fp32 when the caller has computed it.  out_proj False: the normed, gated heads [T, H vdim] come back unprojected."""
+        s = self.spec
+        if proj is None:
+            proj = hops.dense_linear(h, self.w_in, self.b_in, out_dtype=torch.float32)
+        o, den = hops.memory_scan(proj, self.qo, self.ko, self.vo, self.io, self.fo, s.gate_cap, s.dim ** -0.5, s.den_eps, s.heads, s.dim, s.vdim, batch.row_start,
+                                  batch.slot, batch.first_pos, state, mstate, plans=batch.plans, max_rows=batch.max_rows)
+        o = hops.head_norm(o, s.heads, s.vdim, self.norm, self.eps, proj, self.go, gate_act="sigmoid", den=den)
+        return hops.dense_linear(o, self.w_o, out_dtype=torch.float32) if out_proj else o
+
+
+def state_shapes(mixer):
+    """Per-slot shapes of a recurrent mixer's state tensors."""
+    return mixer.state_shapes() if hasattr(mixer, "state_shapes") else [mixer.state_shape()]
+
+
 class ParallelMixer:
     """Two mixers side by side on the same input: left_scale * left(h) + right_scale * right(h).  Each side is any mixer of this module whose
     forward takes `proj` (its input projections as columns of a shared linear): all projections of h, of both sides, are ONE linear.  The
     layer's cache is the sides' caches one after the other (pages for an attention side, a state slot for a recurrent side).  forward returns
-    the two sides' outputs with their scales, (left, left_scale, right, right_scale): the sum is formed by the kernel that ends the sublayer."""
+    the two sides' outputs with their scales, (left, left_scale, right, right_scale): the sum is formed by the kernel that ends the sublayer.
+    out_norms (left [W], right [W]): each side's output is RMS-normed over the width under its weight before it is scaled, by that kernel as well."""
 
-    def __init__(self, left, right, left_scale: float, right_scale: float):
+    def __init__(self, left, right, left_scale: float, right_scale: float, out_norms=None):
         self.left, self.right, self.left_scale, self.right_scale = left, right, float(left_scale), float(right_scale)
+        self.out_norms = tuple(t.contiguous() for t in out_norms) if out_norms is not None else None
         for m in (left, right):
             if getattr(m, "w_in", None) is None or not hasattr(m, "cache_kind"):
                 raise ValueError(f"parallel mixer: {type(m).__name__} cannot run beside another mixer")
@@ -521,8 +655,8 @@ class ParallelMixer:
         left.w_in = right.w_in = None                                            # live on as rows of the shared weight
 
     def cache_parts(self):
-        """Per side: how many cache tensors its forward takes (2: key and value pages; 1: a state)."""
-        return [2 if m.cache_kind() in ("kv", "kv_from") else 1 for m in (self.left, self.right)]
+        """Per side: how many cache tensors its forward takes (key and value pages; or its states)."""
+        return [2 if m.cache_kind() in ("kv", "kv_from") else len(state_shapes(m)) for m in (self.left, self.right)]
 
     def forward(self, h: torch.Tensor, batch: StepBatch, *cache):
         nl_c, _ = self.cache_parts()
@@ -553,25 +687,25 @@ class RouterSpec:
     top: int
     groups: int = 1                      # experts form `groups` runs of neighbours ...
     keep: int = 1                        # ... and only those of the `keep` best runs can be chosen
-    score: str = "softmax"               # "softmax" over the logits | "sigmoid" of each logit
+    score: str = "softmax"               # "softmax" over the logits | "sigmoid" of each logit | "softmax_chosen": softmax over the chosen logits alone
     group_top: int = 1                   # a run scores as its best expert (1) or as the sum of its two best (2)
     scale: float = 1.0                   # the chosen experts weigh score * scale
 
 
 class RoutedExperts:
-    """Mixture of gated experts down_e(act(gate_e h) * up_e h): fp32 softmax router, group-limited top-k, the chosen experts' outputs weighted
+    """Mixture of gated experts down_e(act(gate_e h) * up_e h) or plain ones down_e(act(up_e h)): fp32 softmax router, group-limited top-k, the chosen experts' outputs weighted
     by their softmax scores (not renormalised), plus an optional shared expert that every token runs.  The (token, choice) pairs are sorted
     by expert on the device and each projection of all experts is one grouped linear; nothing returns to the host."""
 
     def __init__(self, router: RouterSpec, w_router: torch.Tensor, gates, ups, downs, shared: Optional["GatedMLP"] = None, act: str = "silu",
                  act_param: float = 0.0, shared_gate: Optional[torch.Tensor] = None):
-        """act_param: the activation's parameter (the limit of "swiglu_clamp").  shared_gate [1, W]: the shared expert's output is multiplied by
+        """gates None: plain experts down_e(act(up_e h)).  act_param: the activation's parameter (the limit of "swiglu_clamp").  shared_gate [1, W]: the shared expert's output is multiplied by
         sigmoid(shared_gate . h), one number per token; its row rides behind the router's in one linear."""
         r = self.router = router
-        if r.score not in ("softmax", "sigmoid") or r.group_top not in (1, 2):
+        if r.score not in ("softmax", "sigmoid", "softmax_chosen") or r.group_top not in (1, 2):
             raise ValueError(f"experts: router score {r.score!r}, groups ranked by their best {r.group_top}")
-        if len(gates) != r.experts or w_router.shape[0] != r.experts:
-            raise ValueError(f"experts: router of {w_router.shape[0]}, {len(gates)} experts, config says {r.experts}")
+        if len(ups) != r.experts or w_router.shape[0] != r.experts:
+            raise ValueError(f"experts: router of {w_router.shape[0]}, {len(ups)} experts, config says {r.experts}")
         if r.experts % r.groups or not 1 <= r.keep <= r.groups or not 1 <= r.top <= (r.experts // r.groups) * r.keep:
             raise ValueError(f"experts: {r.experts} experts in {r.groups} groups, keep {r.keep}, top {r.top}")
         self.w_router = w_router.contiguous()
@@ -582,15 +716,16 @@ class RoutedExperts:
             pad = torch.zeros((-(r.experts + 1)) % 4, w_router.shape[1], dtype=w_router.dtype, device=w_router.device)
             self.w_router = torch.cat([w_router, shared_gate.reshape(1, -1), pad], 0).contiguous()
         self.shared_gated = shared_gate is not None
-        ff, K = gates[0].shape
+        ff, K = ups[0].shape
         pad = (-ff) % 32
         gu, dn = [], []
-        for g, u, d in zip(gates, ups, downs):
+        self.gated = gates is not None
+        for g, u, d in zip(gates if self.gated else [None] * r.experts, ups, downs):
             if pad:
-                z = torch.zeros(pad, K, dtype=g.dtype, device=g.device)
-                g, u = torch.cat([g, z]), torch.cat([u, z])
+                z = torch.zeros(pad, K, dtype=u.dtype, device=u.device)
+                g, u = torch.cat([g, z]) if self.gated else None, torch.cat([u, z])
                 d = torch.cat([d, torch.zeros(d.shape[0], pad, dtype=d.dtype, device=d.device)], 1)
-            gu.append(hops.group_gate_up(g, u)); dn.append(d)
+            gu.append(hops.group_gate_up(g, u) if self.gated else u); dn.append(d)
         self.w_gate_up, self.w_down = torch.stack(gu).contiguous(), torch.stack(dn).contiguous()
         self.shared, self.act, self.act_param = shared, hops.ACTIVATIONS[act], float(act_param)
 
@@ -604,10 +739,10 @@ class RoutedExperts:
             logits = hops.dense_linear(h, self.w_router, out_dtype=torch.float32)
             if self.shared_gated:
                 logits, sgate = logits[:, :self.n_router], logits[:, self.n_router]
-        ids, wts, offs, src, place, tiles = hops.moe_route_sorted(logits, r.experts, r.groups, r.keep, r.top, sigmoid=r.score == "sigmoid",
+        ids, wts, offs, src, place, tiles = hops.moe_route_sorted(logits, r.experts, r.groups, r.keep, r.top, sigmoid=r.score == "sigmoid", chosen=r.score == "softmax_chosen",
                                                                   group_top=r.group_top, scale=r.scale)
         n = ids.numel()
-        a = hops.dense_grouped(h, self.w_gate_up, offs=offs, gather=src, tiles=tiles, rows=n, gated=True, act=self.act, act_param=self.act_param)
+        a = hops.dense_grouped(h, self.w_gate_up, offs=offs, gather=src, tiles=tiles, rows=n, gated=self.gated, act=self.act, act_param=self.act_param)
         y = hops.dense_grouped(a, self.w_down, offs=offs, tiles=tiles, rows=n, out_dtype=torch.float32)
         parts = hops.MoeSum(y, place, wts, self.shared.forward(h) if self.shared is not None else None, sgate)
         if self.shared_gated and not defer:

@@ -14,6 +14,10 @@ sublayers' outputs, sigmoid-routed clamped experts with a gated shared expert) b
 with a shared expert, fixed-decay recurrence, sink attention), at equal width, depth, heads, expert sizes and vocabulary, and its kernels beside
 the like Pokepel kernels against their rooflines.
 
+`--hybrid-design dupenex` measures the Dupenex member (parallel residual streams, windowed attention with channel gates beside matrix memory, a
+delta rule with a decay per key channel, squared-relu experts) beside the Nudorax member at equal width, depth, heads, vocabulary and feed-forward work,
+and its kernels beside the like Nudorax kernels (the delta rule beside Nepudra's).
+
 Output: one JSON line {"hybrid_bench": {size: {"hybrid": {...}, "qwen2": {...}, "kernels": [...]}}} (with --hybrid-design pokepel:
 {"pokepel": {...}, "nufalorn": {...}, "kernels": [...]})."""
 import json
@@ -244,6 +248,62 @@ def nudorax_weights(cfg, dev, seed=0):
     return w
 
 
+def dupenex_config(s, experts=16, top=4, window=1024, streams=4):
+    """Width, heads and vocabulary of `s`, as many layer RUNS as it has layers (two of the layers run twice); windowed grouped-query attention with the
+    sizes' heads beside matrix memory with the recurrent sizes of Nudorax's lightning sides in every second layer, the channel-decay delta rule with
+    width / 64 heads of 64 x 64 and four taps in the others; mixtures of `experts` plain experts of half the FFN width, `top` of them per token (4 x ff x width
+    multiplications against 3.75 of Nudorax's gated experts with the shared one)."""
+    layers, hd = [], s["hd"]
+    mlp = {"kind": "moe", "expert": {"ff": s["ff"] // 2 // 32 * 32}, "router": {"experts": experts, "top": top}}
+    for i in range(s["layers"] - 2):
+        if i % 2 == 0:
+            left = {"heads": s["heads"], "kv_heads": s["kv"], "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": window}, "rot": {"base": 1e6, "dims": hd}}
+            right = {"heads": s["heads"], "dim": hd // 2, "vdim": hd, "gate_cap": 15.0}
+            layers.append({"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp})
+        else:
+            n = s["width"] // 64
+            layers.append({"type": "channel_delta", "mixer": {"heads": n, "kv_heads": n, "dim": 64, "vdim": 64, "conv": 4}, "mlp": mlp})
+    return {"architecture": "Dupenex", "layers": layers, "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "streams": streams,
+            "loop": {"start": 2, "stop": 4, "times": 2}}
+
+
+def dupenex_weights(cfg, dev, seed=0, rank=64):
+    g = torch.Generator(device=dev).manual_seed(seed)
+    W, S = cfg["width"], cfg["streams"]
+    lin = lambda o, i: (torch.randn(o, i, device=dev, generator=g) * i ** -0.5).bfloat16()
+    vec = lambda n, k=0.1, off=0.0: (torch.randn(n, device=dev, generator=g) * k + off).bfloat16()
+    w = {"embed": torch.randn(cfg["vocab"], W, device=dev, generator=g).bfloat16(), "head": lin(cfg["vocab"], W), "final.norm": vec(W, 0.1, 1.0)}
+    for i, L in enumerate(cfg["layers"]):
+        p, mx, mlp = f"l{i}.", L["mixer"], L["mlp"]
+        w[p + "norm1"], w[p + "norm2"] = vec(W, 0.1, 1.0), vec(W, 0.1, 1.0)
+        for q in ("hc1.", "hc2."):
+            w[p + q + "in"], w[p + q + "out"] = vec(S, 0.1, 1.0 / S), vec(S, 0.1, 1.0)
+            w[p + q + "mix"] = (torch.eye(S, device=dev) * 0.9 + 0.1 / S + vec(S * S, 0.02).float().reshape(S, S)).bfloat16()
+        if L["type"] == "parallel":
+            for side, extra in (("left", ()), ("right", ("i", "f"))):
+                a, q = mx[side], p + f"mix.{side}."
+                H, G, d, dv = a["heads"], a.get("kv_heads", a["heads"]), a["dim"], a["vdim"]
+                for n, (o, k) in {"q": (H * d, W), "k": (G * d, W), "v": (G * dv, W), "g": (H * dv, W), "o": (W, H * dv)}.items():
+                    w[q + n] = lin(o, k)
+                for n in extra:
+                    w[q + n], w[q + n + ".b"] = lin(H, W), vec(H, 1.0, 4.0 if n == "f" else 0.0)
+                w[q + "out"] = vec(W, 0.1, 1.0)
+            w[p + "mix.right.norm"] = vec(mx["right"]["heads"] * mx["right"]["vdim"], 0.1, 1.0)
+        else:
+            H, G, d, dv, q = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"], p + "mix."
+            for n, (o, k) in {"q": (G * d, W), "k": (G * d, W), "v": (H * dv, W), "b": (H, W), "a1": (rank, W), "a2": (H * d, rank), "g1": (rank, W), "g2": (H * dv, rank),
+                              "o": (W, H * dv)}.items():
+                w[q + n] = lin(o, k)
+            for n, c in (("q", G * d), ("k", G * d), ("v", H * dv)):
+                w[q + n + ".conv"] = lin(c, mx["conv"])
+            w[q + "A_log"], w[q + "dt_bias"], w[q + "norm"] = vec(H, 0.5), vec(H * d, 0.5, -3.0), vec(dv, 0.1, 1.0)
+        w[p + "mlp.router"] = lin(mlp["router"]["experts"], W)
+        f = mlp["expert"]["ff"]
+        for j in range(mlp["router"]["experts"]):
+            w[p + f"mlp.e{j}.up"], w[p + f"mlp.e{j}.down"] = lin(f, W), lin(W, f)
+    return w
+
+
 def timed(fn, reps=5, warm=2, graph=False):
     """Seconds per call.  graph: the calls are captured into one HIP graph and the replay is timed, so the figure is the kernels' own
     time and not the host's launch path (what a graph-replayed step pays)."""
@@ -279,7 +339,7 @@ def bench_hybrid_engine(s, dev, prompt, batch, steps, design="nufalorn"):
     from .hybrid import HybridConfig, HybridModel
     from .scheduler import ServingEngine
     make_cfg, make_w = {"pokepel": (pokepel_config, pokepel_weights), "nepudra": (nepudra_config, nepudra_weights),
-                        "nudorax": (nudorax_config, nudorax_weights)}.get(design, (hybrid_config, hybrid_weights))
+                        "nudorax": (nudorax_config, nudorax_weights), "dupenex": (dupenex_config, dupenex_weights)}.get(design, (hybrid_config, hybrid_weights))
     cfg = make_cfg(s)
     model = HybridModel(HybridConfig.from_json(cfg), make_w(cfg, dev), torch.bfloat16, dev)
     eng = ServingEngine(model, max_tokens=batch * (prompt + 8 * (steps + 3) + 128), max_seqs=batch, max_step_tokens=1 << 20)
@@ -822,11 +882,172 @@ def kernel_table_nudorax(s, dev, prompt):
     return rows
 
 
+def kernel_table_dupenex(s, dev, prompt):
+    """Dupenex's kernels at this size beside the like kernels of the Nudorax member (the delta rule beside Nepudra's), against max(bytes / HBM, flops /
+    peak of the unit)."""
+    from . import hybrid_ops as hops
+    rows = []
+    timed_k = lambda fn: timed(fn, reps=10, warm=2, graph=True)
+    g = torch.Generator(device=dev).manual_seed(3)
+    bf = lambda *sh: torch.randn(*sh, device=dev, generator=g).bfloat16()
+    f32 = lambda *sh: torch.randn(*sh, device=dev, generator=g)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)
+    W, H, G, hd = s["width"], s["heads"], s["kv"], s["hd"]
+    cfg, ncfg = dupenex_config(s), nudorax_config(s)
+    S, mlp, dm, window = cfg["streams"], cfg["layers"][0]["mlp"], cfg["layers"][1]["mixer"], cfg["layers"][0]["mixer"]["left"]["mask"]["size"]
+    fe, E, top = mlp["expert"]["ff"], mlp["router"]["experts"], mlp["router"]["top"]
+    nmoe = ncfg["layers"][0]["mlp"]
+    nfe, gr = nmoe["expert"]["ff"], nmoe["router"]["groups"]
+
+    def add(family, name, shape, t, nbytes, flops, peak):
+        roof = max(nbytes / HBM, flops / peak)
+        rows.append({"family": family, "kernel": name, "shape": shape, "us": round(t * 1e6, 1), "roofline_us": round(roof * 1e6, 2),
+                     "x_roofline": round(t / roof, 1)})
+
+    page = 64
+    nblk = (prompt + page - 1) // page + 1
+    bt = torch.arange(nblk, dtype=torch.int32, device=dev).reshape(1, nblk)
+    geom, ngeom = hops.attn_geometry(H, G, hd, hd, hd, 0, 0, page, nblk, nblk), hops.attn_geometry(H, G, hd, hd, hd, 1, 0, page, nblk, nblk)
+    kc, vc, sink = bf(nblk, G, page, hd), bf(nblk, G, page, hd), f32(H)
+    # attention: the same window, a gate per value channel against learned sinks
+    for T_, name in ((prompt, "prefill"), (1, "decode")):
+        pos = torch.arange(T_, dtype=torch.int32, device=dev) if T_ > 1 else i32([prompt - 1])
+        seq = torch.zeros(T_, dtype=torch.int32, device=dev)
+        q = f32(T_, 2 * H * hd)
+        og = q[:, H * hd:]
+        kw = float(sum(min(int(p) + 1, window) for p in pos.tolist()))
+        byt = lambda keys: min(prompt, keys) * G * hd * 2 * 2 + T_ * H * hd * 6
+        shape = f"T={T_} H={H} G={G} hd={hd} ctx={prompt}"
+        if T_ > 1:
+            t0 = torch.arange(0, T_, 16, dtype=torch.int32, device=dev)
+            tn = torch.full_like(t0, 16)
+            t = timed_k(lambda: hops.attn_tiles(q, hd ** -0.5, geom, 0, None, None, pos, seq, bt, t0, tn, kc, vc, H, hd, window=window, out_gate=og))
+            add("dupenex", f"attn_tiles prefill (window {window}, channel gates)", shape, t, byt(prompt) + T_ * H * hd * 4, 4.0 * kw * H * hd, MFMA_BF16)
+            t = timed_k(lambda: hops.attn_tiles(q, hd ** -0.5, ngeom, 0, sink, None, pos, seq, bt, t0, tn, kc, vc, H, hd, window=window))
+            add("nudorax", f"attn_tiles prefill (window {window}, learned sinks)", shape, t, byt(prompt), 4.0 * kw * H * hd, MFMA_BF16)
+        else:
+            t = timed_k(lambda: hops.attn_rows(q, hd ** -0.5, geom, 0, None, None, pos, seq, bt, kc, vc, H, hd, window=window, out_gate=og))
+            add("dupenex", f"attn_rows decode (window {window}, channel gates)", shape, t, byt(window) + H * hd * 4, 4.0 * kw * H * hd, MFMA_BF16)
+            t = timed_k(lambda: hops.attn_rows(q, hd ** -0.5, ngeom, 0, sink, None, pos, seq, bt, kc, vc, H, hd, window=window))
+            add("nudorax", f"attn_rows decode (window {window}, learned sinks)", shape, t, byt(window), 4.0 * kw * H * hd, MFMA_BF16)
+    freq = torch.ones(hd // 2, device=dev) * 1e-3
+    for T_ in (prompt, 8):
+        pos, seq = torch.arange(T_, dtype=torch.int32, device=dev), torch.zeros(T_, dtype=torch.int32, device=dev)
+        qkv, qn_, kn_ = f32(T_, (H + 2 * G) * hd), bf(H * hd), bf(G * hd)
+        nb = T_ * ((H + 2 * G) * hd * 4 + H * hd * 4 + 2 * G * hd * 2)
+        t = timed_k(lambda: hops.attn_prep(qkv, H * hd, (H + G) * hd, geom, freq, None, False, 1e-6, pos, seq, bt, kc, vc))
+        add("dupenex", "attn_prep (turn, page write)", f"T={T_} H={H} G={G}", t, nb, 0, VALU_F32)
+        t = timed_k(lambda: hops.attn_prep(qkv, H * hd, (H + G) * hd, ngeom, freq, None, False, 1e-6, pos, seq, bt, kc, vc, q_norm=qn_, k_norm=kn_, norm_whole=True))
+        add("nudorax", "attn_prep (norm over all heads, turn, page write)", f"T={T_} H={H} G={G}", t, nb, 0, VALU_F32)
+    # recurrences: matrix memory against lightning attention, the delta rules, and the norms behind them
+    d, Hd, dd, taps = hd // 2, dm["heads"], dm["dim"], dm["conv"]
+    for T_, name in ((prompt, "prefill"), (8, "decode b=8")):
+        nseq = 1 if T_ > 8 else 8
+        rs = torch.arange(0, T_ + 1, T_ // nseq, dtype=torch.int32, device=dev)
+        slot, fp = torch.arange(nseq, dtype=torch.int32, device=dev), torch.ones(nseq, dtype=torch.int32, device=dev) * 8
+        seq = torch.repeat_interleave(slot, T_ // nseq)
+        hv = H * hd
+        proj = f32(T_, 2 * H * d + 2 * hv + 2 * H)
+        st, ms = torch.zeros(nseq, H, d * hd + d, device=dev), torch.zeros(nseq, H, (hd + 63) // 64, device=dev)
+        nb, fl, shape = T_ * (2 * H * d + 2 * hv) * 4 + 2 * nseq * H * d * hd * 4, 4.0 * T_ * H * d * hd, f"T={T_} H={H} dim={d} vdim={hd}"
+        t = timed_k(lambda: hops.memory_scan(proj, 0, H * d, 2 * H * d, 2 * H * d + 2 * hv, 2 * H * d + 2 * hv + H, 15.0, d ** -0.5, 1e-6, H, d, hd, rs, slot, fp, st, ms,
+                                             max_rows=T_ // nseq))
+        add("dupenex", f"scan matrix memory {name}", shape, t, nb + T_ * H * 12 + 2 * nseq * H * d * 4, fl, VALU_F32)
+        st2, decay = torch.zeros(nseq, H, d, hd, device=dev), torch.full((H,), 0.97, device=dev)
+        t = timed_k(lambda: hops.scan(hops.SCAN_FIXED_SILU, proj, 0, H * d, 2 * H * d, None, decay, None, 1.0, 1.0, H, d, hd, rs, slot, fp, st2, torch.bfloat16,
+                                      max_rows=T_ // nseq))
+        add("nudorax", f"scan lightning {name}", shape, t, nb, fl, VALU_F32)
+        o, wn, den = f32(T_, hv), bf(hv), f32(T_, H).abs() + 1.0
+        t = timed_k(lambda: hops.head_norm(o, H, hd, wn, 1e-6, proj, 2 * H * d + hv, gate_act="sigmoid", den=den))
+        add("dupenex", f"quotient + head norm (weight, sigmoid gate) {name}", f"T={T_} H={H} vdim={hd}", t, T_ * (hv * 10 + H * 4), 0, VALU_F32)
+        t = timed_k(lambda: hops.head_norm(o, 1, hv, wn, 1e-6, proj, 2 * H * d + hv, gate_act="sigmoid"))
+        add("nudorax", f"norm over all heads (weight, sigmoid gate) {name}", f"T={T_} H={H} vdim={hd}", t, T_ * hv * 10, 0, VALU_F32)
+        gd = Hd * dd
+        C = 3 * gd
+        raw, wc, hist = f32(T_, C + 128 + Hd), bf(C, taps), f32(nseq, taps - 1, C)
+        t = timed_k(lambda: hops.short_conv(raw, C, wc, hist, seq, rs, slot, fp, unit_heads=2 * Hd, query_heads=Hd, dim=dd, qscale=dd ** -0.5, low=(C, 128)))
+        add("dupenex", f"short convolutions + unit heads {name}", f"T={T_} channels={C} taps={taps}", t, T_ * (C * 8 + 128 * 6) + C * taps * 2 + nseq * (taps - 1) * C * 4, 0, VALU_F32)
+        x, z, zb, rate = f32(T_, C) * 0.1, f32(T_, gd), f32(gd), f32(Hd).abs()
+        sd = torch.zeros(nseq, Hd, dd, dd, device=dev)
+        nbd, fld, shape = T_ * 5 * gd * 4 + 2 * nseq * Hd * dd * dd * 4, 8.0 * T_ * Hd * dd * dd, f"T={T_} H={Hd} dim={dd} vdim={dd}"
+        t = timed_k(lambda: hops.channel_delta_scan(x, 0, gd, 2 * gd, z, zb, rate, raw[:, C + 128:], Hd, Hd, dd, dd, rs, slot, fp, sd, raw=raw, hist=hist))
+        add("dupenex", f"channel delta scan {name}", shape, t, nbd + 2 * nseq * (taps - 1) * C * 4, fld, VALU_F32)
+        pn = f32(T_, 5 * gd)
+        t = timed_k(lambda: hops.delta_scan(pn, 0, gd, 2 * gd, 3 * gd, z, 0.6, 1e-6, Hd, dd, dd, rs, slot, fp, sd))
+        add("nepudra", f"delta scan {name}", shape, t, nbd + T_ * gd * 4, fld, VALU_F32)
+        low, wl = bf(T_, 128), bf(2, gd, 64)
+        t = timed_k(lambda: hops.dense_grouped(low, wl, x_step=64, y_step=gd, out_dtype=torch.float32))
+        add("dupenex", f"both low-rank products {name}", f"M={T_} G=2 N={gd} K=64", t, 2 * gd * 64 * 2 + T_ * (128 * 2 + 2 * gd * 4), 4.0 * T_ * gd * 64, MFMA_BF16)
+        w2 = bf(gd, 64)
+        t = timed_k(lambda: hops.dense_linear(low[:, :64], w2, out_dtype=torch.float32))
+        add("nepudra", f"low-rank product {name}", f"M={T_} N={gd} K=64", t, gd * 64 * 2 + T_ * (64 * 2 + gd * 4), 2.0 * T_ * gd * 64, MFMA_BF16)
+    # experts: routing + sorting, both grouped linears, and the end of the sublayer
+    for T_ in (prompt, 8, 1):
+        h, z = bf(T_, W), f32(T_, E) * 2
+        t = timed_k(lambda: hops.moe_route_sorted(z, E, 1, 1, top, chosen=True))
+        add("dupenex", "moe route + sort (softmax over the chosen)", f"T={T_} E={E} top={top}", t, T_ * (E * 4 + top * 16), 0, VALU_F32)
+        t = timed_k(lambda: hops.moe_route_sorted(z, E, gr["count"], gr["keep"], top, sigmoid=True, group_top=2, scale=2.5))
+        add("nudorax", "moe route + sort (sigmoid, groups by two best)", f"T={T_} E={E} top={top}", t, T_ * (E * 4 + top * 16), 0, VALU_F32)
+        ids, wts = hops.moe_route(z, 1, 1, top, chosen=True)
+        offs, src, place, tiles = hops.moe_align(ids, E)
+        n, used = T_ * top, len(set(ids.flatten().tolist()))
+        wu = bf(E, fe, W)
+        t = timed_k(lambda: hops.dense_grouped(h, wu, offs=offs, gather=src, tiles=tiles, rows=n, act=hops.ACT_RELU2))
+        add("dupenex", "dense_grouped experts up (squared relu)", f"M={T_}x{top} E={E} ({used} used) N={fe} K={W}", t, used * fe * W * 2 + n * (W + fe) * 2, 2.0 * n * fe * W, MFMA_BF16)
+        wgu = torch.stack([hops.group_gate_up(bf(nfe, W), bf(nfe, W)) for _ in range(E)]).contiguous()
+        t = timed_k(lambda: hops.dense_grouped(h, wgu, offs=offs, gather=src, tiles=tiles, rows=n, gated=True, act=hops.ACT_SWIGLU_CLAMP, act_param=7.0))
+        add("nudorax", "dense_grouped experts gated (clamped)", f"M={T_}x{top} E={E} ({used} used) N={2 * nfe} K={W}", t, used * 2 * nfe * W * 2 + n * (W + nfe) * 2,
+            2.0 * n * 2 * nfe * W, MFMA_BF16)
+        for fam, f in (("dupenex", fe), ("nudorax", nfe)):
+            a, wdn = bf(n, f), bf(E, W, f)
+            t = timed_k(lambda: hops.dense_grouped(a, wdn, offs=offs, tiles=tiles, rows=n, out_dtype=torch.float32))
+            add(fam, "dense_grouped experts down", f"M={T_}x{top} E={E} ({used} used) N={W} K={f}", t, used * f * W * 2 + n * (f * 2 + W * 4), 2.0 * n * f * W, MFMA_BF16)
+        y, X, x, extra, w1, sgate = f32(n, W), f32(T_, S, W), f32(T_, W), f32(T_, W), bf(W), f32(T_)
+        mix, wr, rd = f32(S, S) * 0.3, f32(S), f32(S)
+        t = timed_k(lambda: hops.streams(X, mix=mix, write=wr, read=rd, moe=hops.MoeSum(y, place, wts), w=w1, eps=1e-6))
+        add("dupenex", f"mixture sum + mix of {S} streams + norm", f"T={T_} top={top} W={W}", t, (n + 2 * S * T_) * W * 4 + T_ * W * 2, 0, VALU_F32)
+        t = timed_k(lambda: hops.branch_norm(x, w1, 1e-6, moe=hops.MoeSum(y, place, wts, extra, sgate), rounded=True))
+        add("nudorax", "mixture sum + gated shared + layer norm + residual", f"T={T_} top={top} W={W}", t, (n + 3 * T_) * W * 4 + T_ * W * 2, 0, VALU_F32)
+    for T_ in (prompt, 8):
+        X, x, a, b, w1, na, nb_ = f32(T_, S, W), f32(T_, W), f32(T_, W), f32(T_, W), bf(W), bf(W), bf(W)
+        mix, wr, rd = f32(S, S) * 0.3, f32(S), f32(S)
+        t = timed_k(lambda: hops.streams(X, mix=mix, write=wr, read=rd, a=a, ca=0.5, na=na, b=b, cb=0.5, nb=nb_, branch_eps=1e-6, w=w1, eps=1e-6))
+        add("dupenex", f"two normed branches + mix of {S} streams + norm", f"M={T_} W={W}", t, stream_bytes(T_, W, 2 * S + 2, 1), 0, VALU_F32)
+        t = timed_k(lambda: hops.branch_norm(x, w1, 1e-6, a=a, ca=1.5, b=b, cb=0.75, rounded=True))
+        add("nudorax", "two branches + layer norm + residual (fp32 stream)", f"M={T_} W={W}", t, stream_bytes(T_, W, 4, 1), 0, VALU_F32)
+        t = timed_k(lambda: hops.streams(X, mix=mix, write=wr, read=rd, a=a, w=w1, eps=1e-6))
+        add("dupenex", f"one branch + mix of {S} streams + norm", f"M={T_} W={W}", t, stream_bytes(T_, W, 2 * S + 1, 1), 0, VALU_F32)
+        t = timed_k(lambda: hops.branch_norm(x, w1, 1e-6, a=a, rounded=True))
+        add("nudorax", "one branch + layer norm + residual (fp32 stream)", f"M={T_} W={W}", t, stream_bytes(T_, W, 3, 1), 0, VALU_F32)
+        ids, table = torch.randint(0, s["vocab"], (T_,), device=dev, dtype=torch.int32), bf(s["vocab"], W)
+        t = timed_k(lambda: hops.streams(X, ids=ids, table=table, read=rd, w=w1, eps=1e-6))
+        add("dupenex", f"embedding into {S} streams + norm", f"M={T_} W={W}", t, T_ * W * (2 + 4 * S + 2), 0, VALU_F32)
+        t = timed_k(lambda: hops.embed_scaled(ids, table, 8.0, rounded=True))
+        add("nudorax", "embedding x scale (stream + rounded copy)", f"M={T_} W={W}", t, T_ * W * (2 + 4 + 2), 0, VALU_F32)
+    rows_ = torch.arange(8, dtype=torch.int32, device=dev)
+    X8, x8, a8, w1 = f32(8, S, W), f32(8, W), f32(8, W), bf(W)
+    mix, wr = f32(S, S) * 0.3, f32(S)
+    t = timed_k(lambda: hops.streams(X8, mix=mix, write=wr, a=a8, rows=rows_, w=w1, eps=1e-6))
+    add("dupenex", f"last mix of {S} streams + norm on gathered rows", f"M=8 W={W}", t, 8 * W * (4 * S + 6), 0, VALU_F32)
+    t = timed_k(lambda: hops.norm_rows(x8, rows_, w1, 1e-6))
+    add("nudorax", "last layer norm on gathered rows", f"M=8 W={W}", t, 8 * W * 6, 0, VALU_F32)
+    # linears: ONE input linear per layer
+    np_, nc, nn = (H + 2 * G) * hd + H * hd + 2 * H * d + 2 * H * hd + 2 * H, 3 * Hd * dd + 128 + Hd, (H + 2 * G) * hd + 2 * H * d + 2 * H * hd
+    for M_ in (prompt, 8, 1):
+        x = bf(M_, W)
+        for fam, nm, N_ in (("dupenex", "parallel", np_), ("dupenex", "delta", nc), ("nudorax", "parallel", nn)):
+            wi = bf(N_, W)
+            t = timed_k(lambda: hops.dense_linear(x, wi, out_dtype=torch.float32))
+            add(fam, f"dense_linear all projections of the input ({nm})", f"M={M_} N={N_} K={W}", t, N_ * W * 2 + M_ * (W * 2 + N_ * 4), 2.0 * M_ * N_ * W, MFMA_BF16)
+    return rows
+
+
 def stream_bytes(T_, W, f32_streams, bf16_streams):
     return T_ * W * (4 * f32_streams + 2 * bf16_streams)
 
 
-KERNEL_TABLES = {"pokepel": (kernel_table_pokepel, "nufalorn"), "nepudra": (kernel_table_nepudra, "nufalorn"), "nudorax": (kernel_table_nudorax, "pokepel")}
+KERNEL_TABLES = {"pokepel": (kernel_table_pokepel, "nufalorn"), "nepudra": (kernel_table_nepudra, "nufalorn"), "nudorax": (kernel_table_nudorax, "pokepel"),
+                 "dupenex": (kernel_table_dupenex, "nudorax")}
 
 
 def run_pokepel(args, dev, sizes, member="pokepel"):

@@ -32,7 +32,7 @@ struct DenseParams {
     // groups (tile kernels, blockIdx.z): group g multiplies its rows by the weight w + g * ws (bias + g * N) and writes columns ys * g + ...
     // of y; it reads x from column xs * g on.  Its rows are all M rows, or rows offs[g] .. offs[g + 1] - 1 of a list sorted by group, whose
     // entry r reads x row gather[r] (identity without gather) and writes y row r.  tiles (with offs): {count, (group, first row) x count}, the
-    // 64-row tiles that hold rows; blockIdx.y indexes this list instead of (blockIdx.z, row tile), so no block is spent on a tile without rows.
+    // 64-row tiles that hold rows; the row tile indexes this list instead of (blockIdx.z, row tile), so no block is spent on a tile without rows.
     int G;
     long long xs, ws, ys;
     const int32_t* offs; const int32_t* gather; const int32_t* tiles;
@@ -40,17 +40,29 @@ struct DenseParams {
     const float* egate; int ldg, goff;
 };
 
-// first row and end of the rows of the block's tile in its group, and the group's operand bases
-struct DnGroup { int m0, rend; long long xo, wo, yo; int bo; };
+// The chip deals consecutive blocks to its eight XCDs in turn, each with an L2 of its own.  The (column tile, row tile) pair of a block is chosen such
+// that an XCD walks a contiguous run of tiles in an order of bands of DN_BAND row tiles, column by column: its blocks share the band's rows of x and read
+// every weight column of the run once.
+constexpr int DN_XCD = 8, DN_BAND = 16;
+__device__ __forceinline__ void dn_block_tile(int gx, int gy, int& bx, int& by) {
+    const int nb = gx * gy, id = blockIdx.y * gridDim.x + blockIdx.x;
+    if (id >= nb) { bx = 0; by = gy; return; }               // a block past the list of tiles
+    const int k = id % DN_XCD, j = k * (nb / DN_XCD) + min(k, nb % DN_XCD) + id / DN_XCD;
+    const int band = j / (gx * DN_BAND), rest = j - band * gx * DN_BAND, h = min(DN_BAND, gy - band * DN_BAND);
+    bx = rest / h; by = band * DN_BAND + rest % h;
+}
+
+// the block's column tile, first row and end of the rows of its tile in its group, and the group's operand bases
+struct DnGroup { int bx, m0, rend; long long xo, wo, yo; int bo; };
 __device__ __forceinline__ DnGroup dn_group(const DenseParams& p, int tile_rows) {
-    int g = blockIdx.z;
+    int g = blockIdx.z, by;
     DnGroup r;
+    dn_block_tile(gridDim.x, p.tiles ? p.tiles[0] : gridDim.y, r.bx, by);
     if (p.tiles) {
-        const int i = blockIdx.y;
-        if (i >= p.tiles[0]) { r.m0 = r.rend = 0; return r; }
-        g = p.tiles[1 + 2 * i]; r.m0 = p.tiles[2 + 2 * i]; r.rend = p.offs[g + 1];
+        if (by >= p.tiles[0]) { r.m0 = r.rend = 0; return r; }
+        g = p.tiles[1 + 2 * by]; r.m0 = p.tiles[2 + 2 * by]; r.rend = p.offs[g + 1];
     } else {
-        r.m0 = (p.offs ? p.offs[g] : 0) + blockIdx.y * tile_rows; r.rend = p.offs ? p.offs[g + 1] : p.M;
+        r.m0 = (p.offs ? p.offs[g] : 0) + by * tile_rows; r.rend = p.offs ? p.offs[g + 1] : p.M;
     }
     r.xo = p.xs * g; r.wo = p.ws * g; r.yo = p.ys * g; r.bo = g * p.N;
     return r;
@@ -107,7 +119,7 @@ __global__ __launch_bounds__(256) void dense_tile_bf16_kernel(DenseParams p) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = wave & 1, wn = wave >> 1;                       // wave tile: rows wm*32.., cols wn*64..
     const DnGroup gr = dn_group(p, TB_M);
-    const int m0 = gr.m0, n0 = blockIdx.x * TB_N;
+    const int m0 = gr.m0, n0 = gr.bx * TB_N;
     if (m0 >= gr.rend) return;
     const bf16* X = (const bf16*)p.x + gr.xo;
     const bf16* W = (const bf16*)p.w + gr.wo;
@@ -202,7 +214,7 @@ __global__ __launch_bounds__(256) void dense_tile_f32_kernel(DenseParams p) {
     __shared__ __attribute__((aligned(16))) float Bs[TF_K * TF_LD];   // [k][n]
     const int tid = threadIdx.x, ty = tid >> 4, tx = tid & 15;
     const DnGroup gr = dn_group(p, TF_M);
-    const int m0 = gr.m0, n0 = blockIdx.x * TF_N;
+    const int m0 = gr.m0, n0 = gr.bx * TF_N;
     if (m0 >= gr.rend) return;
     const float* X = (const float*)p.x + gr.xo;
     const float* W = (const float*)p.w + gr.wo;

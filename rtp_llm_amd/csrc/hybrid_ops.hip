@@ -1377,22 +1377,21 @@ struct ConvParams {
     const int32_t* seq; const int32_t* row_start; const int32_t* slot; const int32_t* first_pos;
     float* out;                                     // [rows, C]
     int lo, R; void* low;                           // low [rows, R] of the activation type (null: none)
+    int piece;                                      // channels of a wave's piece outside the unit heads (at most 256)
 };
-
-constexpr int CONV_PIECE = 256;                     // channels of a wave's piece outside the unit heads
 
 template <typename T>
 __global__ __launch_bounds__(256) void hy_short_conv_kernel(ConvParams p, int pieces_v, int pieces) {
     const int r = blockIdx.x, lane = threadIdx.x & 63, piece = blockIdx.y * 4 + (threadIdx.x >> 6);
     if (piece >= pieces) return;
     if (piece >= p.units + pieces_v) {              // the low-rank inputs
-        const int b = (piece - p.units - pieces_v) * CONV_PIECE;
-        for (int c = b + lane; c < min(b + CONV_PIECE, p.R); c += 64) ((T*)p.low)[(size_t)r * p.R + c] = (T)p.proj[(size_t)r * p.ld + p.lo + c];
+        const int b = (piece - p.units - pieces_v) * p.piece;
+        for (int c = b + lane; c < min(b + p.piece, p.R); c += 64) ((T*)p.low)[(size_t)r * p.R + c] = (T)p.proj[(size_t)r * p.ld + p.lo + c];
         return;
     }
     const bool head = piece < p.units;
-    const int c0 = head ? piece * p.dim : p.units * p.dim + (piece - p.units) * CONV_PIECE;
-    const int c1 = head ? c0 + p.dim : min(c0 + CONV_PIECE, p.C);
+    const int c0 = head ? piece * p.dim : p.units * p.dim + (piece - p.units) * p.piece;
+    const int c1 = head ? c0 + p.dim : min(c0 + p.piece, p.C);
     const int sq = p.seq[r], i = r - p.row_start[sq], pos = p.first_pos[sq] + i, K = p.taps - 1;
     const float* hist = p.hist + (size_t)p.slot[sq] * K * p.C;
     constexpr int NC = 8;                           // channels per lane kept in registers (unit heads of up to 512 channels)
@@ -1419,6 +1418,77 @@ __global__ __launch_bounds__(256) void hy_short_conv_kernel(ConvParams p, int pi
     for (int e = 0; e < NC; ++e) {
         const int c = c0 + lane + 64 * e;
         if (c < c1) p.out[(size_t)r * p.C + c] = v[e] * f;
+    }
+}
+
+// The same for runs of CONV_ROWS rows (prompt portions): a wave keeps its channels' weights and the last taps - 1 inputs in registers and slides over the rows.
+constexpr int CONV_ROWS = 8;
+
+template <typename T, int TAPS, int NC>              // NC: most channels per lane of a piece
+__global__ __launch_bounds__(256) void hy_short_conv_run_kernel(ConvParams p, int rows, int pieces_v, int pieces) {
+    const int ra = blockIdx.x * CONV_ROWS, rb = min(ra + CONV_ROWS, rows), lane = threadIdx.x & 63, piece = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (piece >= pieces) return;
+    if (piece >= p.units + pieces_v) {
+        const int b = (piece - p.units - pieces_v) * p.piece;
+        for (int r = ra; r < rb; ++r)
+            for (int c = b + lane; c < min(b + p.piece, p.R); c += 64) ((T*)p.low)[(size_t)r * p.R + c] = (T)p.proj[(size_t)r * p.ld + p.lo + c];
+        return;
+    }
+    constexpr int K = TAPS - 1;
+    const bool head = piece < p.units;
+    const int c0 = head ? piece * p.dim : p.units * p.dim + (piece - p.units) * p.piece;
+    const int c1 = head ? c0 + p.dim : min(c0 + p.piece, p.C);
+    float w[NC][TAPS], x[CONV_ROWS][NC], old[K > 0 ? K : 1][NC];     // old[j]: the input K - j tokens before the current one
+#pragma unroll
+    for (int e = 0; e < NC; ++e) {
+        const int c = c0 + lane + 64 * e;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[e][j] = c < c1 ? (float)((const T*)p.w)[(size_t)c * TAPS + j] : 0.f;
+#pragma unroll
+        for (int u = 0; u < CONV_ROWS; ++u) x[u][e] = (c < c1 && ra + u < rb) ? p.proj[(size_t)(ra + u) * p.ld + c] : 0.f;
+    }
+    const float qs = piece < p.uq ? p.qscale : 1.f;
+#pragma unroll
+    for (int u = 0; u < CONV_ROWS; ++u) {
+        const int r = ra + u;
+        if (r >= rb) break;
+        const int sq = p.seq[r], i = r - p.row_start[sq];
+        if (u == 0 || i == 0) {                          // the run's or the sequence's first row: earlier inputs from rows before the run or from the slot
+            const int pos = p.first_pos[sq] + i;
+            const float* hist = p.hist + (size_t)p.slot[sq] * K * p.C;
+#pragma unroll
+            for (int j = 0; j < K; ++j)
+#pragma unroll
+                for (int e = 0; e < NC; ++e) {
+                    const int c = c0 + lane + 64 * e, back = K - j;
+                    float v = 0.f;
+                    if (c < c1) {
+                        if (back <= i) v = p.proj[(size_t)(r - back) * p.ld + c];
+                        else if (back <= pos) v = hist[(size_t)(K + i - back) * p.C + c];
+                    }
+                    old[j][e] = v;
+                }
+        }
+        float v[NC], ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < NC; ++e) {
+            float a = 0.f;
+#pragma unroll
+            for (int j = 0; j < K; ++j) a = __builtin_fmaf(w[e][j], old[j][e], a);
+            a = __builtin_fmaf(w[e][K], x[u][e], a);
+            v[e] = hy_silu(a);
+            ss = __builtin_fmaf(v[e], v[e], ss);
+#pragma unroll
+            for (int j = 0; j + 1 < K; ++j) old[j][e] = old[j + 1][e];
+            if (K > 0) old[K > 0 ? K - 1 : 0][e] = x[u][e];
+        }
+        float f = 1.f;
+        if (head) f = 1.f / sqrtf(hy_wave_sum(ss) + p.unit_eps) * qs;
+#pragma unroll
+        for (int e = 0; e < NC; ++e) {
+            const int c = c0 + lane + 64 * e;
+            if (c < c1) p.out[(size_t)r * p.C + c] = v[e] * f;
+        }
     }
 }
 
@@ -1456,7 +1526,12 @@ struct DeltaParams {
     const float* raw; int ldr, C, taps; float* hist;
 };
 
-__device__ __forceinline__ float hy_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// exp, log1p of a value in (0, 1], softplus and sigmoid from the hardware's exp2 / log2 / reciprocal (each within about an ulp): the gates of a pass are formed
+// by every block of a head, and a walk with one wave per SIMD pays for each instruction
+__device__ __forceinline__ float hy_fexp(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896340736f); }
+__device__ __forceinline__ float hy_flog1p(float e) { return e < 1e-3f ? e * (1.f - e * (0.5f - e * 0.33333334f)) : __builtin_amdgcn_logf(1.f + e) * 0.69314718055994530942f; }
+__device__ __forceinline__ float hy_fsoftplus(float z) { return fmaxf(z, 0.f) + hy_flog1p(hy_fexp(-fabsf(z))); }
+__device__ __forceinline__ float hy_fsigmoid(float z) { return __builtin_amdgcn_rcpf(1.f + hy_fexp(-z)); }
 
 template <int LPC> __device__ __forceinline__ float hy_lanes_sum(float v);
 template <> __device__ __forceinline__ float hy_lanes_sum<4>(float v) {
@@ -1488,6 +1563,10 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
     }
     float fr[EL], fk[EL], fa[EL], fz[EL], fv[VE];
     const int kvh = CHANNEL ? h / (p.H / p.G) : h;
+    const float rate = CHANNEL ? p.rate[h] : 0.f;
+    float zb[EL];                                     // decay bias of the thread's channels (the same channels every pass)
+#pragma unroll
+    for (int e = 0; e < EL; ++e) { const int d = (tid + e * 256) % dpad; zb[e] = (CHANNEL && d < p.dim) ? p.zbias[h * p.dim + d] : 0.f; }
     auto fetch = [&](int t0) {
         const int nt = min(TOK, r1 - t0);
 #pragma unroll
@@ -1499,7 +1578,7 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
                 const int hd = h * p.dim + d;
                 if constexpr (CHANNEL) {
                     fr[e] = row[p.ro + kvh * p.dim + d]; fk[e] = row[p.ko + kvh * p.dim + d]; fa[e] = p.bp[(size_t)(t0 + t) * p.ldb + h];
-                    fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd] + p.zbias[hd];
+                    fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd] + zb[e];
                 } else {
                     fr[e] = row[p.ro + hd]; fk[e] = row[p.ko + hd]; fa[e] = row[p.ao + hd];
                     fz[e] = p.z[(size_t)(t0 + t) * p.ldz + hd];
@@ -1521,8 +1600,8 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
             if (i >= nt * dpad) continue;
             const bool in = d < p.dim;                  // rows beyond the key size: zero keys, no removal, state stays zero
             if constexpr (CHANNEL) {
-                const float g = in ? expf(-p.rate[h] * hy_softplus(fz[e])) : 1.f;
-                r_s[i] = fr[e]; w_s[i] = g; u_s[i] = g * fk[e]; b_s[i] = in ? hy_sigmoid(fa[e]) * fk[e] : 0.f;
+                const float g = in ? hy_fexp(-rate * hy_fsoftplus(fz[e])) : 1.f;
+                r_s[i] = fr[e]; w_s[i] = g; u_s[i] = g * fk[e]; b_s[i] = in ? hy_fsigmoid(fa[e]) * fk[e] : 0.f;
                 continue;
             }
             r_s[i] = fr[e]; k_s[i] = fk[e];
@@ -2296,8 +2375,19 @@ extern "C" int mi355_hy_short_conv(const float* proj, int32_t ld, int32_t rows, 
     MI355_CHECK_ARG(proj && w && seq && row_start && slot && first_pos && out && rows > 0 && C > 0 && taps > 0 && (hist || taps == 1), "hy_short_conv: bad argument");
     MI355_CHECK_ARG(units >= 0 && uq >= 0 && uq <= units && units * dim <= C && (units == 0 || (dim > 0 && dim <= 512)), "hy_short_conv: %d heads of %d in %d channels", units, dim, C);
     MI355_CHECK_ARG(ld >= C && (!low || (R > 0 && lo >= 0 && ld >= lo + R)), "hy_short_conv: ld=%d lo=%d R=%d", ld, lo, R);
-    const ConvParams p{proj, ld, C, taps, w, units, uq, dim, qscale, unit_eps, hist, seq, row_start, slot, first_pos, out, lo, R, low};
-    const int pv = (C - units * dim + CONV_PIECE - 1) / CONV_PIECE, pieces = units + pv + (low ? (R + CONV_PIECE - 1) / CONV_PIECE : 0);
+    const int nc = dim <= 64 ? 1 : dim <= 128 ? 2 : 4;
+    const ConvParams p{proj, ld, C, taps, w, units, uq, dim, qscale, unit_eps, hist, seq, row_start, slot, first_pos, out, lo, R, low, 64 * nc};
+    const int pv = (C - units * dim + p.piece - 1) / p.piece, pieces = units + pv + (low ? (R + p.piece - 1) / p.piece : 0);
+    if (rows > 128 && taps >= 2 && taps <= 4 && dim <= 256) {
+        const dim3 grid((rows + CONV_ROWS - 1) / CONV_ROWS, (pieces + 3) / 4);
+#define HY_CONV(TAPS_, NC_) HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_short_conv_run_kernel<T, TAPS_, NC_>), grid, dim3(256), 0, (hipStream_t)stream, p, rows, pv, pieces))
+#define HY_CONV_T(TAPS_) do { if (nc == 1) HY_CONV(TAPS_, 1); else if (nc == 2) HY_CONV(TAPS_, 2); else HY_CONV(TAPS_, 4); } while (0)
+        if (taps == 2) HY_CONV_T(2); else if (taps == 3) HY_CONV_T(3); else HY_CONV_T(4);
+#undef HY_CONV_T
+#undef HY_CONV
+        MI355_CHECK_LAUNCH("hy_short_conv_run_kernel");
+        return MI355_OK;
+    }
     HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_short_conv_kernel<T>, dim3(rows, (pieces + 3) / 4), dim3(256), 0, (hipStream_t)stream, p, pv, pieces));
     MI355_CHECK_LAUNCH("hy_short_conv_kernel");
     return MI355_OK;

@@ -1184,7 +1184,9 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
     float s[RD];
     const bool fresh = p.first_pos[sq] == 0;
     // MEM: the block of the first value columns also carries n, row d = ds * RD + c of it in lane c < RD of wave ds
-    __shared__ float keep_s[16], take_s[16], em_s[16];
+    // (e^(-m) has two buffers taken in turns: it is read after a pass's walk, when the first wave may already form the next pass's gates)
+    __shared__ float keep_s[16], take_s[16], em_s[2][16];
+    int turn = 0;
     const bool own_n = MEM && v0 == 0 && c < RD;
     float n = 0.f, P = 1.f, m_run = 0.f, ri = 0.f, rf = 0.f, re = 0.f;
     if constexpr (MEM) {
@@ -1229,7 +1231,7 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
         }
     };
     if (r0 < r1) fetch(r0);
-    for (int t0 = r0; t0 < r1; t0 += TOK) {
+    for (int t0 = r0; t0 < r1; t0 += TOK, turn ^= 1) {
         const int nt = min(TOK, r1 - t0);
         if constexpr (MEM) {
             if (tid < 64) {
@@ -1245,7 +1247,7 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
                     keep = expf(lf + prev - m); take = expf(li - m); em = expf(-m);
                     m_run = __shfl(m, nt - 1, 64);
                 }
-                if (tid < nt) { keep_s[tid] = keep; take_s[tid] = take; em_s[tid] = em; }
+                if (tid < nt) { keep_s[tid] = keep; take_s[tid] = take; em_s[turn][tid] = em; }
             }
             __syncthreads();
         }
@@ -1342,7 +1344,7 @@ __global__ __launch_bounds__(1024) void hy_scan_kernel(ScanParams p) {
                     float* dp = p.mem.den + (size_t)(t0 + t) * p.H + h;
                     if (c == 0) {
                         if (p.apply) nq += *dp;
-                        *dp = p.mem.raw ? nq : fmaxf(fabsf(nq), em_s[t]) + p.mem.den_eps;
+                        *dp = p.mem.raw ? nq : fmaxf(fabsf(nq), em_s[turn][t]) + p.mem.den_eps;
                     }
                 }
         }

@@ -7,7 +7,8 @@
 // helpers: PolyNorm, and routing / sorting / weighted sum of a mixture of experts.  Options of the attention kernels: sliding window, tanh
 // cap on the scores, per-head sigmoid gate on the output, normed queries and keys, scaled rotary magnitude, a query temperature.  For members
 // whose sublayers follow each other: the layer's end as residual update + weighted average over the results of all earlier layers + norm,
-// and a hashed bigram row beside the token embedding.
+// and a hashed bigram row beside the token embedding.  For members with several residual streams: their mixing, write-back, weighted sum and norm in one
+// launch; short causal convolutions; a delta rule with a decay per key channel; a matrix memory under exponential gates.
 //
 // One ragged batch of rows serves prefill portions and decode tokens alike: every row carries its position and the index of its
 // sequence; a sequence carries its block-table row, its state slot and the range of its rows.  What the model states as 32-bit is fp32

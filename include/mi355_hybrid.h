@@ -150,6 +150,27 @@ int mi355_hy_attn_tiles_ex2(const float* q, int32_t ldq, float scale, const int3
                             int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, float softcap, const float* ogate,
                             int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream);
 
+/* A window that keeps the first tokens of a sequence, latent attention whose queries come from a projection of their own (pair layout as an argument), and
+ * a loop over layers whose passes start from a linear of [stream; embedding output]. */
+int mi355_hy_attn_rows_ex3(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                           const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache, const void* vcache,
+                           void* out, int32_t splits, float* parts, int32_t window, int32_t keep, float softcap, const float* ogate, int32_t ldg,
+                           int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_attn_tiles_ex3(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                            const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0, const int32_t* tile_n,
+                            int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, int32_t keep, float softcap,
+                            const float* ogate, int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_latent_prep_ex(const float* q, int32_t ldq, const float* down, int32_t ldd, const int32_t* geom, int32_t layout, const float* freq, float mag,
+                            const void* cw, float eps, const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, void* qn,
+                            float* qabs, void* cache, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_head_norm_ex3(const float* o, int32_t ldo, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg,
+                           int32_t goff, void* out, int32_t w_heads, int32_t gate_sigmoid, const float* den, int32_t act_dtype, mi355_stream_t stream);
+int mi355_hy_residual_round(float* x, const float* a, const float* b, const float* gate, int32_t ldg, float mult, int32_t n, int32_t W, void* raw,
+                            int32_t ldraw, const float* moe_y, const int32_t* moe_place, const float* moe_wts, int32_t moe_top, int32_t act_dtype,
+                            mi355_stream_t stream);
+int mi355_hy_embed_scaled_ex(const int32_t* ids, int32_t rows, const void* table, int32_t W, int32_t vocab, float scale, float* out, void* outh,
+                             int32_t ldh, int32_t act_dtype, mi355_stream_t stream);
+
 #ifdef __cplusplus
 }
 #endif

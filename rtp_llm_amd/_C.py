@@ -207,6 +207,12 @@ HYBRID_SIGNATURES = {
     "mi355_hy_attn_rows_ex2": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, f32, vp, i32, i32, i32, vp]),
     "mi355_hy_attn_tiles_ex2": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, f32, vp, i32, i32, i32, vp]),
     "mi355_hy_branch_norm": (i32, [vp, vp, f32, vp, f32, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, vp, i32, f32, vp, i32, vp]),
+    "mi355_hy_attn_rows_ex3": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, f32, vp, i32, i32, i32, vp]),
+    "mi355_hy_attn_tiles_ex3": (i32, [vp, i32, f32, ip, i32, vp, vp, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32, i32, f32, vp, i32, i32, i32, vp]),
+    "mi355_hy_latent_prep_ex": (i32, [vp, i32, vp, i32, ip, i32, vp, f32, vp, f32, vp, vp, vp, i32, vp, vp, vp, i32, vp]),
+    "mi355_hy_head_norm_ex3": (i32, [vp, i32, i32, i32, i32, vp, f32, vp, i32, i32, vp, i32, i32, vp, i32, vp]),
+    "mi355_hy_residual_round": (i32, [vp, vp, vp, vp, i32, f32, i32, i32, vp, i32, vp, vp, vp, i32, i32, vp]),
+    "mi355_hy_embed_scaled_ex": (i32, [vp, i32, vp, i32, i32, f32, vp, vp, i32, i32, vp]),
 }
 
 _lib = None

@@ -8,7 +8,8 @@
 // cap on the scores, per-head sigmoid gate on the output, normed queries and keys, scaled rotary magnitude, a query temperature.  For members
 // whose sublayers follow each other: the layer's end as residual update + weighted average over the results of all earlier layers + norm,
 // and a hashed bigram row beside the token embedding.  For members with several residual streams: their mixing, write-back, weighted sum and norm in one
-// launch; short causal convolutions; a delta rule with a decay per key channel; a matrix memory under exponential gates.
+// launch; short causal convolutions; a delta rule with a decay per key channel; a matrix memory under exponential gates.  For layers that run in a loop
+// fed with the embedding output: the stream's rounded copy beside it, the operand of the linear in front of every pass.
 //
 // One ragged batch of rows serves prefill portions and decode tokens alike: every row carries its position and the index of its
 // sequence; a sequence carries its block-table row, its state slot and the range of its rows.  What the model states as 32-bit is fp32
@@ -98,12 +99,14 @@ template <> __device__ __forceinline__ void hy_store4<bf16>(bf16* p, const float
 // x[src] <- x[src] + mult * (ga * a[src] + gb * b[src]) (written back unless rows are gathered), then h1 = norm(x) * (off + w1), h2 likewise.
 // gate null: ga = gb = 1; else ga = sigmoid(gate[src, c]) and gb = sigmoid(gate[src, W + c]) (fp32 pre-activations, row stride ldg).
 // ms.y non-null: the second branch is a mixture's weighted sum formed here, b[src] (if any) + sum_k ms.wts[src, k] * ms.y[ms.place[src, k]].
+// raw non-null: the new rows themselves, rounded to the activation type, go to raw (row stride ldraw); without h1 and h2 nothing is normed.
 // VEC: W % 4 == 0, four channels per thread and trip (16-byte accesses on the fp32 stream).
 struct MoeSum { const float* y; const int32_t* place; const float* wts; int top; };
 
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void hy_residual_norm_kernel(float* x, const float* a, const float* b, MoeSum ms, const float* gate, int ldg, float mult,
-                                                               const int32_t* rows, const T* w1, const T* w2, float off, float eps, int W, T* h1, T* h2) {
+                                                               const int32_t* rows, const T* w1, const T* w2, float off, float eps, int W, T* h1, T* h2,
+                                                               T* raw, int ldraw) {
     extern __shared__ __attribute__((aligned(16))) float hy_xs[];
     __shared__ float red[4];
     const int r = blockIdx.x, src = rows ? rows[r] : r;
@@ -141,9 +144,11 @@ __global__ __launch_bounds__(256) void hy_residual_norm_kernel(float* x, const f
             for (int e = 0; e < V; ++e) v[e] = v[e] + mult * (ya[e] + yb[e]);
             if (!rows) { if (VEC) hy_store4<float>(x + i, v); else x[i] = v[0]; }
         }
+        if (raw) { if (VEC) hy_store4<T>(raw + (size_t)r * ldraw + c, v); else raw[(size_t)r * ldraw + c] = (T)v[0]; }
 #pragma unroll
         for (int e = 0; e < V; ++e) { hy_xs[c + e] = v[e]; ss = __builtin_fmaf(v[e], v[e], ss); }
     }
+    if (!h1 && !h2) return;
     ss = hy_wave_sum(ss);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
     __syncthreads();
@@ -168,17 +173,17 @@ __global__ __launch_bounds__(256) void hy_residual_norm_kernel(float* x, const f
 }
 
 // ------------------------------------------------------------------------------------------------ scaled embedding; norm on a sublayer's OUTPUT
-// out[r] = table[ids[r]] * scale (fp32 stream); outh (null: none): the same rows rounded to the activation type, the input of the first sublayer of a
-// stack whose sublayers read the stream itself.
+// out[r] = table[ids[r]] * scale (fp32 stream); outh (null: none, row stride ldh): the same rows rounded to the activation type, the input of the first
+// sublayer of a stack whose sublayers read the stream itself, or the part of a wider row that a later linear reads again.
 template <typename T>
-__global__ __launch_bounds__(256) void hy_embed_scaled_kernel(const int32_t* ids, const T* table, int W, int vocab, float scale, float* out, T* outh) {
+__global__ __launch_bounds__(256) void hy_embed_scaled_kernel(const int32_t* ids, const T* table, int W, int vocab, float scale, float* out, T* outh, int ldh) {
     const int r = blockIdx.x;
     int id = ids[r];
     id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
     for (int c = threadIdx.x; c < W; c += 256) {
         const float v = (float)table[(size_t)id * W + c] * scale;
         out[(size_t)r * W + c] = v;
-        if (outh) outh[(size_t)r * W + c] = (T)v;
+        if (outh) outh[(size_t)r * ldh + c] = (T)v;
     }
 }
 
@@ -599,7 +604,8 @@ __device__ __forceinline__ float hy_lane_f(float v, int j) { return __builtin_bi
 // softcap > 0: score <- softcap tanh(score / softcap) after the scale; ogate non-null: head h of row r is multiplied by
 // sigmoid(ogate[r * ldg + h]) (fp32 pre-activations, one number per head).
 // (gate_channels: one number per value channel instead, ogate[r * ldg + h * vdim + c]).
-struct AttnExtra { int window; float softcap; const float* ogate; int ldg; int gate_channels; };
+// keep (with window > 0): the keys j < keep of a sequence stay visible to every row behind them, whatever their distance.
+struct AttnExtra { int window; float softcap; const float* ogate; int ldg; int gate_channels; int keep; };
 __device__ __forceinline__ float hy_channel_gate(const AttnExtra& ex, int r, int h, int vdim, int c) {
     return ex.gate_channels ? hy_sigmoid(ex.ogate[(size_t)r * ex.ldg + h * vdim + c]) : 1.f;
 }
@@ -622,7 +628,8 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
     const int32_t* bt = block_table + (size_t)seq[r] * g.max_blocks;
     for (int d = tid; d < g.dim; d += NT) q_s[d] = q[(size_t)r * ldq + h * g.dim + d];
     __syncthreads();
-    const int lo = hy_first_visible(p, chunk, ex.window);
+    // the visible keys as one run of `nvis` indices: the kept first tokens in front of the window, then the window
+    const int lo = hy_first_visible(p, chunk, ex.window), kept = ex.window > 0 ? min(ex.keep, lo) : 0, nvis = kept + p - lo + 1;
     // the sink is a key of (unscaled) score sink[h] that carries no value: wave 0 starts from m = sink[h], l = 1
     float m = (sink && wave == 0 && sp == 0) ? sink[h] : -INFINITY, l = (sink && wave == 0 && sp == 0) ? 1.f : 0.f;
     float acc[NV], facc[8];
@@ -643,8 +650,8 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
     float qv[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) qv[i] = (coop && kl_ok) ? q_s[kl * 8 + i] : 0.f;
-    for (int t0 = lo + (sp * NW + wave) * 64; t0 <= p; t0 += 64 * NW * S) {
-        const int kj = t0 + lane;
+    for (int t0 = (sp * NW + wave) * 64; t0 < nvis; t0 += 64 * NW * S) {
+        const int kj = t0 + lane < kept ? t0 + lane : t0 + lane - kept + lo;
         const bool valid = kj <= p;
         float s = -INFINITY;
         int rowi = 0;                                              // row of the key inside the cache tensors: (page * G + kv head) * page size + offset
@@ -652,7 +659,7 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
         if (coop) {
             // LK lanes share a key row (8 channels = one 16- or 32-byte piece each), so a load instruction reads KK whole rows instead of one
             // piece of 64 rows; the partial products are summed over the LK lanes and handed to the lane that owns the key
-            const int nk = min(64, p - t0 + 1);
+            const int nk = min(64, nvis - t0);
             float sc = 0.f;
             constexpr int UB = 8;                                  // load instructions in flight
             for (int it0 = 0; it0 * KK < nk; it0 += UB) {
@@ -689,7 +696,7 @@ __global__ __launch_bounds__(1024) void hy_attn_rows_kernel(const float* q, int 
         const float corr = (m == -INFINITY) ? 0.f : expf(m - mn);
         l = l * corr + hy_wave_sum(pj);
         m = mn;
-        const int nv = min(64, p - t0 + 1);
+        const int nv = min(64, nvis - t0);
         if (fast) {
             // LPK lanes share one key's value row (8 channels = 16 bytes each), so one load instruction covers KPI keys
 #pragma unroll
@@ -898,10 +905,13 @@ __global__ __launch_bounds__(256) void hy_attn_tiles_kernel(const float* q, int 
     for (int cb = 0; cb < NCBM; ++cb) o[cb] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int plast = p0 + n - 1;
     const int rlo_last = hy_first_visible(plast, chunk, ex.window);
-    int rlo4[4];                                              // first visible position of the lane's four rows
-#pragma unroll
-    for (int e = 0; e < 4; ++e) rlo4[e] = hy_first_visible(p0 + lq * 4 + e, chunk, ex.window);
     const int kstart = hy_first_visible(p0, chunk, ex.window) & ~31;
+    // with kept first tokens: the steps that hold those in front of kstart come first (what else they hold is masked)
+    const int keep = ex.window > 0 ? ex.keep : 0, nkept = (min(keep, kstart) + 31) >> 5, nsteps = nkept + ((plast - kstart) >> 5) + 1;
+    unsigned gap4[4];                                         // hidden keys between the kept ones and the window of the lane's four rows: keep .. keep + gap - 1
+#pragma unroll
+    for (int e = 0; e < 4; ++e) gap4[e] = (unsigned)max(hy_first_visible(p0 + lq * 4 + e, chunk, ex.window) - keep, 0);
+    auto step_key = [&](int st) { return (st < nkept ? 0 : kstart - 32 * nkept) + 32 * st; };
     // the key fragments and raw value rows of the next 32 keys are fetched while the current 32 are worked on
     bf16x8 kn[2][DKM];
     u32x4 vn[VEM];
@@ -922,8 +932,9 @@ __global__ __launch_bounds__(256) void hy_attn_tiles_kernel(const float* q, int 
             }
         }
     };
-    fetch(kstart);
-    for (int t0 = kstart; t0 <= plast; t0 += 32) {
+    fetch(step_key(0));
+    for (int st = 0; st < nsteps; ++st) {
+        const int t0 = step_key(st);
         f32x4 s[2];
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb) {
@@ -956,19 +967,19 @@ __global__ __launch_bounds__(256) void hy_attn_tiles_kernel(const float* q, int 
                 }
             }
         }
-        if (t0 + 32 <= plast) fetch(t0 + 32);                  // in flight during the softmax and the second product
+        if (st + 1 < nsteps) fetch(step_key(st + 1));          // in flight during the softmax and the second product
         // a step whose 32 keys are visible to every row of the tile (behind the first row, inside the last row's block) needs no mask
-        const bool interior = t0 + 31 <= p0 && t0 >= rlo_last;
+        const bool interior = t0 + 31 <= p0 && (t0 >= rlo_last || t0 + 32 <= keep);
         // mask, running maximum, weights; fragment element e is row 4 lq + e, the lane's key columns are kb * 16 + lr
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int row = lq * 4 + e, rpos = p0 + row;
-            const int rlo = rlo4[e];
+            const unsigned gap = gap4[e];
             float sv[2];
 #pragma unroll
             for (int kb = 0; kb < 2; ++kb) {
                 const int kpos = t0 + kb * 16 + lr;
-                sv[kb] = (interior || (row < n && kpos <= rpos && kpos >= rlo)) ? s[kb][e] : -INFINITY;
+                sv[kb] = (interior || (row < n && kpos <= rpos && (unsigned)(kpos - keep) >= gap)) ? s[kb][e] : -INFINITY;
             }
             const float mn = fmaxf(m[e], hy_max16(fmaxf(sv[0], sv[1])));
             float pw[2] = {0.f, 0.f}, corr = 1.f;
@@ -1705,11 +1716,11 @@ __global__ __launch_bounds__(256) void hy_delta_kernel(DeltaParams p) {
 // gate (silu, or gate_sigmoid: sigmoid); den non-null: the head is divided by den[row * H + h] first: one block per (row, head), a single wave for heads of up to 256 channels and a wave per 256 channels
 // beyond, up to sixteen (one "head" that spans all heads of a row: a norm over the whole concatenation)
 template <typename T>
-__global__ __launch_bounds__(1024) void hy_head_norm_kernel(const float* o, int H, int vdim, const T* w, float eps, const float* gate, int ldg, int goff, T* out,
+__global__ __launch_bounds__(1024) void hy_head_norm_kernel(const float* o, int ldo, int H, int vdim, const T* w, float eps, const float* gate, int ldg, int goff, T* out,
                                                            int w_heads, int gate_sigmoid, const float* den) {
     __shared__ float red[16];
     const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, NT = blockDim.x;
-    const float* src = o + ((size_t)r * H + h) * vdim;
+    const float* src = o + (size_t)r * ldo + (size_t)h * vdim;
     const float sc = den ? 1.f / den[(size_t)r * H + h] : 1.f;
     float ss = 0.f;
     for (int c = tid; c < vdim; c += NT) { const float v = src[c] * sc; ss = __builtin_fmaf(v, v, ss); }
@@ -1732,21 +1743,35 @@ __global__ __launch_bounds__(1024) void hy_head_norm_kernel(const float* o, int 
 
 // ------------------------------------------------------------------------------------------------ latent attention: normed latent + shared rotated key -> page; queries split
 // A token caches ONE row [c (R) | rotated shared key part (dr) | zeros up to dpad] for all heads: c = unit-RMS(first R outputs of the down
-// projection) * w, the key part is the remaining dr outputs with their first `rdims` channels turned by the position (interleaved pairs,
+// projection) * w, the key part is the remaining dr outputs with their first `rdims` channels turned by the position (pair layout as hy_pair,
 // cos and sin times `mag`).  Values are the first R channels of the same row.  Per query head the un-rotated part goes to qn (activation
 // type, input of the per-head product with the key up-projection) and the rotated part to columns R.. of the head's absorbed query row
 // (fp32, dpad wide, zeros behind).
-struct LatentGeom { int H, dim, dr, R, dpad, rdims, page, max_blocks, num_pages; };
+// The query heads (q, row stride ldq) and the down projection (down, ldd) may be columns of one buffer or come from two.
+struct LatentGeom { int H, dim, dr, R, dpad, rdims, page, max_blocks, num_pages, layout; };
+
+// channel j of src's first rdims channels after the turn
+__device__ __forceinline__ float hy_turned(const float* src, int j, int rdims, int layout, float fp, const float* freq, float mag) {
+    const int half = rdims / 2, pr = layout == 0 ? j >> 1 : (j < half ? j : j - half);
+    const bool second = layout == 0 ? (j & 1) : j >= half;
+    int c0, c1;
+    hy_pair(layout, pr, rdims, c0, c1);
+    float sn, cs;
+    sincosf(fp * freq[pr], &sn, &cs);
+    sn *= mag; cs *= mag;
+    const float u = src[c0], w = src[c1];
+    return second ? (w * cs + u * sn) : (u * cs - w * sn);
+}
 
 template <typename T>
-__global__ __launch_bounds__(256) void hy_latent_prep_kernel(const float* proj, int ld, int doff, LatentGeom g, const float* freq, float mag, const T* cw, float eps,
+__global__ __launch_bounds__(256) void hy_latent_prep_kernel(const float* q, int ldq, const float* down, int ldd, LatentGeom g, const float* freq, float mag, const T* cw, float eps,
                                                              const int32_t* pos, const int32_t* seq, const int32_t* block_table, T* qn, float* qabs, T* cache) {
     __shared__ float red[4];
     const int r = blockIdx.x, tid = threadIdx.x;
     const int p = pos[r];
     const float fp = (float)p;
-    const float* row = proj + (size_t)r * ld;
-    const int hd = g.dim + g.dr, hp = g.rdims / 2;
+    const float* row = q + (size_t)r * ldq;
+    const int hd = g.dim + g.dr;
     // queries
     for (int i = tid; i < g.H * g.dim; i += 256) qn[(size_t)r * g.H * g.dim + i] = (T)row[(i / g.dim) * hd + i % g.dim];
     const int tail = g.dpad - g.R;                                   // rotated part + padding of an absorbed query row
@@ -1755,23 +1780,15 @@ __global__ __launch_bounds__(256) void hy_latent_prep_kernel(const float* proj, 
         float v = 0.f;
         if (j < g.dr) {
             const float* qr = row + h * hd + g.dim;
-            if (j < g.rdims) {
-                const int pr = j >> 1;
-                float sn, cs;
-                sincosf(fp * freq[pr], &sn, &cs);
-                sn *= mag; cs *= mag;
-                const float u = qr[2 * pr], w = qr[2 * pr + 1];
-                v = (j & 1) ? (w * cs + u * sn) : (u * cs - w * sn);
-            } else v = qr[j];
+            v = j < g.rdims ? hy_turned(qr, j, g.rdims, g.layout, fp, freq, mag) : qr[j];
         }
         qabs[((size_t)r * g.H + h) * g.dpad + g.R + j] = v;
     }
-    (void)hp;
     // cache row
     bool ok = p >= 0 && p / g.page < g.max_blocks;
     int pg = 0;
     if (ok) { pg = block_table[(size_t)seq[r] * g.max_blocks + p / g.page]; ok = pg >= 0 && pg < g.num_pages; }
-    const float* dk = row + doff;
+    const float* dk = down + (size_t)r * ldd;
     float ss = 0.f;
     for (int c = tid; c < g.R; c += 256) ss = __builtin_fmaf(dk[c], dk[c], ss);
     ss = hy_wave_sum(ss);
@@ -1785,14 +1802,7 @@ __global__ __launch_bounds__(256) void hy_latent_prep_kernel(const float* proj, 
         if (c < g.R) v = dk[c] * inv * (float)cw[c];
         else if (c < g.R + g.dr) {
             const int j = c - g.R;
-            if (j < g.rdims) {
-                const int pr = j >> 1;
-                float sn, cs;
-                sincosf(fp * freq[pr], &sn, &cs);
-                sn *= mag; cs *= mag;
-                const float u = dk[g.R + 2 * pr], w = dk[g.R + 2 * pr + 1];
-                v = (j & 1) ? (w * cs + u * sn) : (u * cs - w * sn);
-            } else v = dk[c];
+            v = j < g.rdims ? hy_turned(dk + g.R, j, g.rdims, g.layout, fp, freq, mag) : dk[c];
         }
         dst[c] = (T)v;
     }
@@ -2052,6 +2062,25 @@ extern "C" int mi355_hy_embed_bigram(const int32_t* ids, int32_t rows, const voi
     return MI355_OK;
 }
 
+static int hy_residual(float* x, const float* a, const float* b, const MoeSum& ms, const float* gate, int32_t ldg, float mult, const int32_t* rows, int32_t n, int32_t W,
+                       const void* w1, const void* w2, float weight_offset, float eps, void* h1, void* h2, void* raw, int32_t ldraw, int32_t act_dtype,
+                       mi355_stream_t stream) {
+    MI355_CHECK_ARG(!ms.y || (ms.place && ms.wts && ms.top > 0), "hy_residual_norm: a mixture's sum needs its places and weights");
+    MI355_CHECK_ARG(x && n > 0 && W > 0 && (!h1 || w1) && (!h2 || w2), "hy_residual_norm: n=%d W=%d", n, W);
+    MI355_CHECK_ARG((size_t)W * 4 <= 64 * 1024, "hy_residual_norm: W=%d too wide for one block", W);
+    MI355_CHECK_ARG(!gate || ldg >= 2 * W, "hy_residual_norm: gate row stride %d for two gates of %d", ldg, W);
+    MI355_CHECK_ARG(!raw || (ldraw >= W && !rows), "hy_residual_norm: rounded rows at stride %d", ldraw);
+    auto al = [](const void* p_) { return ((uintptr_t)p_ & 15) == 0; };
+    if (W % 4 == 0 && ldg % 4 == 0 && ldraw % 4 == 0 && al(x) && al(a) && al(b) && al(gate) && al(w1) && al(w2) && al(h1) && al(h2) && al(ms.y) && al(raw))
+        HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_residual_norm_kernel<T, true>), dim3(n), dim3(256), (size_t)W * 4, (hipStream_t)stream, x, a, b, ms, gate, ldg,
+                                                  mult, rows, (const T*)w1, (const T*)w2, weight_offset, eps, W, (T*)h1, (T*)h2, (T*)raw, ldraw));
+    else
+        HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_residual_norm_kernel<T, false>), dim3(n), dim3(256), (size_t)W * 4, (hipStream_t)stream, x, a, b, ms, gate, ldg,
+                                                  mult, rows, (const T*)w1, (const T*)w2, weight_offset, eps, W, (T*)h1, (T*)h2, (T*)raw, ldraw));
+    MI355_CHECK_LAUNCH("hy_residual_norm_kernel");
+    return MI355_OK;
+}
+
 // x [*, W] fp32 stream; a, b [*, W] fp32 branch outputs (either may be null); rows: null, or `n` source rows to gather (x is then read only).
 // h1 / h2 [n, W] of act_dtype: x / rms(x) * (weight_offset + w).  w2 / h2 may be null.
 // gate: null, or fp32 [*, ldg] pre-activations of per-channel branch gates: a is scaled by sigmoid(gate[:, 0:W]), b by sigmoid(gate[:, W:2W]).
@@ -2061,20 +2090,17 @@ extern "C" int mi355_hy_gated_residual_norm(float* x, const float* a, const floa
                                             int32_t n, int32_t W, const void* w1, const void* w2, float weight_offset, float eps, void* h1, void* h2,
                                             const float* moe_y, const int32_t* moe_place, const float* moe_wts, int32_t moe_top, int32_t act_dtype,
                                             mi355_stream_t stream) {
-    MI355_CHECK_ARG(!moe_y || (moe_place && moe_wts && moe_top > 0), "hy_residual_norm: a mixture's sum needs its places and weights");
-    const MoeSum ms{moe_y, moe_place, moe_wts, moe_top};
-    MI355_CHECK_ARG(x && n > 0 && W > 0 && (!h1 || w1) && (!h2 || w2), "hy_residual_norm: n=%d W=%d", n, W);
-    MI355_CHECK_ARG((size_t)W * 4 <= 64 * 1024, "hy_residual_norm: W=%d too wide for one block", W);
-    MI355_CHECK_ARG(!gate || ldg >= 2 * W, "hy_residual_norm: gate row stride %d for two gates of %d", ldg, W);
-    auto al = [](const void* p_) { return ((uintptr_t)p_ & 15) == 0; };
-    if (W % 4 == 0 && ldg % 4 == 0 && al(x) && al(a) && al(b) && al(gate) && al(w1) && al(w2) && al(h1) && al(h2) && al(moe_y))
-        HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_residual_norm_kernel<T, true>), dim3(n), dim3(256), (size_t)W * 4, (hipStream_t)stream, x, a, b, ms, gate, ldg,
-                                                  mult, rows, (const T*)w1, (const T*)w2, weight_offset, eps, W, (T*)h1, (T*)h2));
-    else
-        HY_DISPATCH(act_dtype, hipLaunchKernelGGL((hy_residual_norm_kernel<T, false>), dim3(n), dim3(256), (size_t)W * 4, (hipStream_t)stream, x, a, b, ms, gate, ldg,
-                                                  mult, rows, (const T*)w1, (const T*)w2, weight_offset, eps, W, (T*)h1, (T*)h2));
-    MI355_CHECK_LAUNCH("hy_residual_norm_kernel");
-    return MI355_OK;
+    return hy_residual(x, a, b, MoeSum{moe_y, moe_place, moe_wts, moe_top}, gate, ldg, mult, rows, n, W, w1, w2, weight_offset, eps, h1, h2, nullptr, 0, act_dtype, stream);
+}
+
+// The same update of the stream without a norm: raw (act_dtype, row stride ldraw) receives the new rows rounded to the activation type, the operand of a
+// linear that reads the stream itself.
+extern "C" int mi355_hy_residual_round(float* x, const float* a, const float* b, const float* gate, int32_t ldg, float mult, int32_t n, int32_t W, void* raw,
+                                       int32_t ldraw, const float* moe_y, const int32_t* moe_place, const float* moe_wts, int32_t moe_top, int32_t act_dtype,
+                                       mi355_stream_t stream) {
+    MI355_CHECK_ARG(raw != nullptr, "hy_residual_round: no output");
+    return hy_residual(x, a, b, MoeSum{moe_y, moe_place, moe_wts, moe_top}, gate, ldg, mult, nullptr, n, W, nullptr, nullptr, 0.f, 0.f, nullptr, nullptr, raw, ldraw,
+                       act_dtype, stream);
 }
 
 extern "C" int mi355_hy_residual_norm(float* x, const float* a, const float* b, float mult, const int32_t* rows, int32_t n, int32_t W,
@@ -2086,9 +2112,15 @@ extern "C" int mi355_hy_residual_norm(float* x, const float* a, const float* b, 
 // out fp32 [rows, W] = table[ids] * scale; outh (act_dtype [rows, W], or null): the same rows in the activation type.
 extern "C" int mi355_hy_embed_scaled(const int32_t* ids, int32_t rows, const void* table, int32_t W, int32_t vocab, float scale, float* out, void* outh,
                                      int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(ids && table && out && rows > 0 && W > 0 && vocab > 0, "hy_embed_scaled: rows=%d W=%d", rows, W);
+    return mi355_hy_embed_scaled_ex(ids, rows, table, W, vocab, scale, out, outh, W, act_dtype, stream);
+}
+
+// outh has a row stride of its own (ldh).
+extern "C" int mi355_hy_embed_scaled_ex(const int32_t* ids, int32_t rows, const void* table, int32_t W, int32_t vocab, float scale, float* out, void* outh,
+                                        int32_t ldh, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(ids && table && out && rows > 0 && W > 0 && vocab > 0 && (!outh || ldh >= W), "hy_embed_scaled: rows=%d W=%d ldh=%d", rows, W, ldh);
     HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_embed_scaled_kernel<T>, dim3(rows), dim3(256), 0, (hipStream_t)stream, ids, (const T*)table, W, vocab, scale, out,
-                                              (T*)outh));
+                                              (T*)outh, ldh));
     MI355_CHECK_LAUNCH("hy_embed_scaled_kernel");
     return MI355_OK;
 }
@@ -2235,9 +2267,18 @@ extern "C" int mi355_hy_attn_rows_ex2(const float* q, int32_t ldq, float scale, 
                                       const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache,
                                       const void* vcache, void* out, int32_t splits, float* parts, int32_t window, float softcap, const float* ogate,
                                       int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(geom && window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
-                    "hy_attn_rows: window=%d chunk=%d ldg=%d", window, chunk, ldg);
-    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels};
+    return mi355_hy_attn_rows_ex3(q, ldq, scale, geom, chunk, sink, vfreq, pos, seq, block_table, rows, kcache, vcache, out, splits, parts, window, 0, softcap, ogate, ldg,
+                                  gate_channels, act_dtype, stream);
+}
+
+// keep > 0 (with a window): the keys j < keep of the sequence stay visible to every row at or behind them.
+extern "C" int mi355_hy_attn_rows_ex3(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                                      const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, const void* kcache,
+                                      const void* vcache, void* out, int32_t splits, float* parts, int32_t window, int32_t keep, float softcap,
+                                      const float* ogate, int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(geom && window >= 0 && keep >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
+                    "hy_attn_rows: window=%d keep=%d chunk=%d ldg=%d", window, keep, chunk, ldg);
+    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels, keep};
     MI355_CHECK_ARG(q && geom && pos && seq && block_table && kcache && vcache && out && rows > 0 && chunk >= 0, "hy_attn_rows: bad argument");
     MI355_CHECK_ARG(splits >= 1 && splits <= 64 && (splits == 1 || parts), "hy_attn_rows: %d splits", splits);
     MI355_CHECK_ARG(!vfreq || geom[3] % 2 == 0, "hy_attn_rows: rotated values need an even value size (%d)", geom[3]);
@@ -2276,9 +2317,18 @@ extern "C" int mi355_hy_attn_tiles_ex2(const float* q, int32_t ldq, float scale,
                                        const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0,
                                        const int32_t* tile_n, int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, float softcap,
                                        const float* ogate, int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(geom && window >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
-                    "hy_attn_tiles: window=%d chunk=%d ldg=%d", window, chunk, ldg);
-    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels};
+    return mi355_hy_attn_tiles_ex3(q, ldq, scale, geom, chunk, sink, vfreq, pos, seq, block_table, tile_row0, tile_n, tiles, kcache, vcache, out, window, 0, softcap, ogate,
+                                   ldg, gate_channels, act_dtype, stream);
+}
+
+// keep as in mi355_hy_attn_rows_ex3.
+extern "C" int mi355_hy_attn_tiles_ex3(const float* q, int32_t ldq, float scale, const int32_t* geom, int32_t chunk, const float* sink, const float* vfreq,
+                                       const int32_t* pos, const int32_t* seq, const int32_t* block_table, const int32_t* tile_row0,
+                                       const int32_t* tile_n, int32_t tiles, const void* kcache, const void* vcache, void* out, int32_t window, int32_t keep,
+                                       float softcap, const float* ogate, int32_t ldg, int32_t gate_channels, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(geom && window >= 0 && keep >= 0 && (window == 0 || chunk == 0) && softcap >= 0.f && (!ogate || ldg >= geom[0] * (gate_channels ? geom[3] : 1)) && (ogate || !gate_channels),
+                    "hy_attn_tiles: window=%d keep=%d chunk=%d ldg=%d", window, keep, chunk, ldg);
+    const AttnExtra ex{window, softcap, ogate, ldg, gate_channels, keep};
     MI355_CHECK_ARG(q && geom && pos && seq && block_table && tile_row0 && tile_n && kcache && vcache && out && tiles > 0 && chunk >= 0, "hy_attn_tiles: bad argument");
     const AttnGeom g{geom[0], geom[1], geom[2], geom[3], geom[4], geom[5], geom[6], geom[7], geom[8], geom[9], geom[10] > 0 ? geom[10] : geom[3]};
     if (int e = hy_geom_ok(g)) return e;
@@ -2474,8 +2524,15 @@ extern "C" int mi355_hy_head_norm_ex(const float* o, int32_t rows, int32_t H, in
 extern "C" int mi355_hy_head_norm_ex2(const float* o, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg,
                                       int32_t goff, void* out, int32_t w_heads, int32_t gate_sigmoid, const float* den, int32_t act_dtype,
                                       mi355_stream_t stream) {
-    MI355_CHECK_ARG(o && out && rows > 0 && H > 0 && vdim > 0, "hy_head_norm: bad argument");
-    HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_head_norm_kernel<T>, dim3(rows, H), dim3(vdim > 256 ? std::min(1024, (vdim + 255) / 256 * 64) : 64), 0, (hipStream_t)stream, o, H, vdim, (const T*)w, eps,
+    return mi355_hy_head_norm_ex3(o, H * vdim, rows, H, vdim, w, eps, gate, ldg, goff, out, w_heads, gate_sigmoid, den, act_dtype, stream);
+}
+
+// o has a row stride of its own (ldo): the heads may be columns of a wider buffer.
+extern "C" int mi355_hy_head_norm_ex3(const float* o, int32_t ldo, int32_t rows, int32_t H, int32_t vdim, const void* w, float eps, const float* gate, int32_t ldg,
+                                      int32_t goff, void* out, int32_t w_heads, int32_t gate_sigmoid, const float* den, int32_t act_dtype,
+                                      mi355_stream_t stream) {
+    MI355_CHECK_ARG(o && out && rows > 0 && H > 0 && vdim > 0 && ldo >= H * vdim, "hy_head_norm: bad argument");
+    HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_head_norm_kernel<T>, dim3(rows, H), dim3(vdim > 256 ? std::min(1024, (vdim + 255) / 256 * 64) : 64), 0, (hipStream_t)stream, o, ldo, H, vdim, (const T*)w, eps,
                                               gate, ldg, goff, (T*)out, w_heads, gate_sigmoid, den));
     MI355_CHECK_LAUNCH("hy_head_norm_kernel");
     return MI355_OK;
@@ -2487,12 +2544,22 @@ extern "C" int mi355_hy_head_norm_ex2(const float* o, int32_t rows, int32_t H, i
 extern "C" int mi355_hy_latent_prep(const float* proj, int32_t ld, int32_t doff, const int32_t* geom, const float* freq, float mag, const void* cw, float eps,
                                     const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, void* qn, float* qabs, void* cache,
                                     int32_t act_dtype, mi355_stream_t stream) {
-    MI355_CHECK_ARG(proj && geom && cw && pos && seq && block_table && qn && qabs && cache && rows > 0, "hy_latent_prep: null argument");
-    const LatentGeom g{geom[0], geom[1], geom[2], geom[3], geom[4], geom[5], geom[6], geom[7], geom[8]};
+    MI355_CHECK_ARG(proj && geom && ld >= doff + geom[3] + geom[2] && doff >= geom[0] * (geom[1] + geom[2]), "hy_latent_prep: ld=%d doff=%d", ld, doff);
+    return mi355_hy_latent_prep_ex(proj, ld, proj + doff, ld, geom, 0, freq, mag, cw, eps, pos, seq, block_table, rows, qn, qabs, cache, act_dtype, stream);
+}
+
+// Queries (fp32 [rows, ldq], H heads of dim + dr) and down projection (fp32 [rows, ldd], R + dr) from buffers of their own; layout: the pairs of the
+// rotation (0 interleaved, 1 half a span apart).
+extern "C" int mi355_hy_latent_prep_ex(const float* q, int32_t ldq, const float* down, int32_t ldd, const int32_t* geom, int32_t layout, const float* freq, float mag,
+                                       const void* cw, float eps, const int32_t* pos, const int32_t* seq, const int32_t* block_table, int32_t rows, void* qn,
+                                       float* qabs, void* cache, int32_t act_dtype, mi355_stream_t stream) {
+    MI355_CHECK_ARG(q && down && geom && cw && pos && seq && block_table && qn && qabs && cache && rows > 0, "hy_latent_prep: null argument");
+    const LatentGeom g{geom[0], geom[1], geom[2], geom[3], geom[4], geom[5], geom[6], geom[7], geom[8], layout};
     MI355_CHECK_ARG(g.H > 0 && g.dim > 0 && g.dr >= 0 && g.R > 0 && g.dpad >= g.R + g.dr && g.rdims >= 0 && g.rdims <= g.dr && g.rdims % 2 == 0 && (g.rdims == 0 || freq),
                     "hy_latent_prep: heads=%d dim=%d rot=%d rank=%d padded=%d span=%d", g.H, g.dim, g.dr, g.R, g.dpad, g.rdims);
-    MI355_CHECK_ARG(g.page > 0 && g.max_blocks > 0 && g.num_pages > 0 && ld >= doff + g.R + g.dr && doff >= g.H * (g.dim + g.dr), "hy_latent_prep: ld=%d doff=%d", ld, doff);
-    HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_latent_prep_kernel<T>, dim3(rows), dim3(256), 0, (hipStream_t)stream, proj, ld, doff, g, freq, mag, (const T*)cw, eps,
+    MI355_CHECK_ARG(g.page > 0 && g.max_blocks > 0 && g.num_pages > 0 && ldd >= g.R + g.dr && ldq >= g.H * (g.dim + g.dr) && (layout == 0 || layout == 1),
+                    "hy_latent_prep: ldq=%d ldd=%d layout=%d", ldq, ldd, layout);
+    HY_DISPATCH(act_dtype, hipLaunchKernelGGL(hy_latent_prep_kernel<T>, dim3(rows), dim3(256), 0, (hipStream_t)stream, q, ldq, down, ldd, g, freq, mag, (const T*)cw, eps,
                                               pos, seq, block_table, (T*)qn, qabs, (T*)cache));
     MI355_CHECK_LAUNCH("hy_latent_prep_kernel");
     return MI355_OK;

@@ -26,7 +26,11 @@ every run with a cache or state of its own; mixers: a delta rule with a decay pe
 with an elementwise output gate beside a matrix memory under exponential gates, both normed before they are added; silu-gated MLPs and
 mixtures of plain squared-relu experts weighted by the softmax over the chosen logits; checkpoint tensors l<i>.mix.{q, k, v (+ .conv), b, A_log, a1,
 a2, dt_bias, g1, g2, norm, o}, l<i>.mix.left.{q, k, v, g, o, out}, l<i>.mix.right.{q, k, v, g, i, f (+ .b), norm, o, out}, l<i>.mlp.{gate, up, down} or
-l<i>.mlp.{router, e<j>.{up, down}})."""
+l<i>.mlp.{router, e<j>.{up, down}}) and Kerotar (parallel layers x <- x + mixer(h) + mlp(h) under one plain norm over a scaled embedding; a span of layers
+runs several times in a row, every pass starting from x <- A [x; embedding output] + s_pass (loop.in, loop.step); mixers: sliding-window attention that
+keeps the first tokens, with a learned sink and queries / keys normed over all heads at once, and latent attention with a latent for the queries too and a
+gate per head; clamped gated MLPs and mixtures of silu-gated experts weighted over the chosen; checkpoint tensors l<i>.mix.{q, k, v, q.norm, k.norm,
+sink, o} or l<i>.mix.{dq, dq.norm, uq, dkv, dkv.norm, uk, uv, g, o}, l<i>.mlp.{gate, up, down} or l<i>.mlp.{router, e<j>.{gate, up, down}})."""
 import json
 import os
 from dataclasses import dataclass, field
@@ -94,6 +98,7 @@ class HybridConfig:
     out_norm: bool = False                           # sequential layers whose sublayers read the stream ITSELF and whose OUTPUT is normed: x <- x + norm(f(x))
     streams: int = 0                                 # > 0: the residual is this many parallel streams mixed at every sublayer (sequential layers)
     loop: Optional[Tuple[int, int, int]] = None      # (start, stop, times): layers start .. stop - 1 run `times` times in a row with the same weights
+    loop_input: bool = False                         # every pass of the loop starts from x <- A [x; x0] + s_pass, x0 the embedding output (loop.in, loop.step)
     norm_kind: str = "rms"                           # "rms" | "layer" (mean removed, variance of the deviations, a weight and no bias)
 
     def layer_runs(self) -> List[int]:
@@ -105,6 +110,13 @@ class HybridConfig:
         if not 0 <= start <= stop <= n or times < 0:
             raise ValueError(f"loop: layers {start} .. {stop - 1} of {n}, {times} times")
         return list(range(start)) + list(range(start, stop)) * times + list(range(stop, n))
+
+    def pass_starts(self) -> Dict[int, int]:
+        """Place in layer_runs() of a pass's first layer -> number of the pass."""
+        if self.loop is None or self.loop[0] == self.loop[1]:
+            return {}
+        start, stop, times = self.loop
+        return {start + t * (stop - start): t for t in range(times)}
 
     @staticmethod
     def from_json(cfg: dict) -> "HybridConfig":
@@ -300,8 +312,47 @@ def dupenex_from_json(cfg: dict) -> HybridConfig:
     return c
 
 
+def kerotar_from_json(cfg: dict) -> HybridConfig:
+    """The Kerotar reading of config.json.  Layer types: "attention" (mixer.{heads, kv_heads, dim, vdim, scale, mask.{size, keep_first}, rot.{dims, base}}:
+    sliding window that keeps the first tokens, a learned sink, queries and keys normed over all heads at once) and "latent_attention" (mixer.{heads, dim,
+    rot_dim, vdim, kv_rank, scale, rot.{dims, base}}: a latent for the queries, whose size is that of its weight, a gate per head, no sink); rotary pairs are
+    half a span apart in both.  mlp: null, {kind: dense, ff, limit} (clamped gated) or {kind: moe, expert.ff, router.{experts, top}} (silu-gated experts; the
+    chosen experts' softmax scores divided by their sum, which is the softmax over the chosen logits).  embedding.scale; loop.{start, stop, times}."""
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        kind, mx, mlp = L["type"], L["mixer"], L.get("mlp")
+        if kind == "attention":
+            mask = mx.get("mask") or {}
+            spec = AttentionSpec(heads=int(mx["heads"]), kv_heads=int(mx.get("kv_heads") or mx["heads"]), dim=int(mx["dim"]), vdim=int(mx.get("vdim") or mx["dim"]),
+                                 scale=float(mx["scale"]), rot=RotarySpec.from_json(mx.get("rot"), "halves"), window=int(mask.get("size") or 0),
+                                 keep_first=int(mask.get("keep_first") or 0), sink=True, learned_sink=True, qk_norm=True, qk_norm_whole=True)
+        elif kind == "latent_attention":
+            rot = dict(mx.get("rot") or {})
+            rot.setdefault("dims", mx["rot_dim"])
+            spec = LatentAttentionSpec(heads=int(mx["heads"]), dim=int(mx["dim"]), rot_dim=int(mx["rot_dim"]), vdim=int(mx.get("vdim") or mx["dim"]),
+                                       kv_rank=int(mx["kv_rank"]), scale=float(mx["scale"]), rot=RotarySpec.from_json(rot if "base" in rot else None, "halves"),
+                                       sink=False, gate_channels=False, query_latent=True)
+        else:
+            raise NotImplementedError(f"layer {i}: mixer type {kind!r}")
+        if mlp is None:
+            layers.append(HybridLayerSpec(kind, spec))
+        elif mlp.get("kind", "dense") == "dense":
+            layers.append(HybridLayerSpec(kind, spec, int(mlp["ff"]), "swiglu_clamp", act_param=float(mlp["limit"])))
+        elif mlp["kind"] == "moe":
+            r = mlp["router"]
+            layers.append(HybridLayerSpec(kind, spec, int(mlp["expert"]["ff"]), "silu", "experts", RouterSpec(int(r["experts"]), int(r["top"]), score="softmax_chosen")))
+        else:
+            raise NotImplementedError(f"layer {i}: mlp kind {mlp.get('kind')!r}")
+    loop = cfg.get("loop")
+    c = HybridConfig(name=str(cfg["architecture"]), vocab=int(cfg["vocab"]), width=int(cfg["width"]), layers=layers, eps=float(cfg["norm"]["eps"]), norm_offset=0.0,
+                     shared_norm=True, embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+                     loop=(int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else None, loop_input=bool(loop))
+    c.layer_runs()                                       # the loop's span is checked here
+    return c
+
+
 _READERS = {"nufalorn": HybridConfig.nufalorn_from_json, "pokepel": HybridConfig.pokepel_from_json, "nepudra": nepudra_from_json, "nudorax": nudorax_from_json,
-            "dupenex": dupenex_from_json}
+            "dupenex": dupenex_from_json, "kerotar": kerotar_from_json}
 
 
 class HybridModel:
@@ -378,7 +429,9 @@ class HybridModel:
             elif L.kind == "delta_rule":
                 mixer = GeneralizedDeltaRule(L.mixer, sub(p + "mix.", ["r", "k", "v", "a", "a.b", "g", "w1", "w2", "w0", "norm", "o"]), cfg.eps)
             elif L.kind == "latent_attention":
-                mixer = LatentAttention(L.mixer, sub(p + "mix.", ["q", "dkv", "dkv.norm", "uk", "uv", "sink", "g", "o"]), cfg.eps, page, self.device)
+                a = L.mixer
+                names = (["dq", "dq.norm", "uq"] if a.query_latent else ["q"]) + ["dkv", "dkv.norm", "uk", "uv", "o"] + (["sink"] if a.sink else []) + (["g"] if a.out_gate else [])
+                mixer = LatentAttention(a, sub(p + "mix.", names), cfg.eps, page, self.device)
             elif L.kind == "retention":
                 mixer = Retention(L.mixer, sub(p + "mix.", ["q", "k", "v", "g", "o"]), cfg.eps, self.device)
             elif L.kind == "hgrn2":
@@ -389,7 +442,7 @@ class HybridModel:
             if L.ff is not None:
                 gated = lambda q, act, par=0.0: GatedMLP(get(q + "gate"), get(q + "up"), get(q + "down"), act, par)
                 if L.mlp_kind == "gated":
-                    mlp = gated(p + "mlp.", L.mlp_act)
+                    mlp = gated(p + "mlp.", L.mlp_act, L.act_param)
                 elif L.mlp_kind == "polynorm":
                     mlp = PolyNormMLP(get(p + "mlp.up"), get(p + "mlp.down"), tensors[p + "mlp.act"], cfg.eps)
                 else:
@@ -406,24 +459,35 @@ class HybridModel:
                 if mlp is None:                        # the kernel reads two gates per row: keep the row stride at 2 W
                     gate_w = torch.cat([gate_w, torch.zeros_like(gate_w)], 0).contiguous()
                     gate_b = torch.cat([gate_b, torch.zeros_like(gate_b)], 0).contiguous()
-                if isinstance(mlp, RoutedExperts):     # the router's logits come out of the same linear: columns [2W, 2W + experts), padded to 4
-                    E = L.router.experts
-                    rw = torch.cat([mlp.w_router, torch.zeros((-E) % 4, cfg.width, dtype=dtype, device=self.device)], 0)
-                    gate_w = torch.cat([gate_w, rw], 0).contiguous()
+            # one norm feeds both branches: the router's logits come out of a linear shared with other projections of h (rows padded to 4)
+            if cfg.shared_norm and isinstance(mlp, RoutedExperts) and not mlp.shared_gated:
+                rw = torch.cat([mlp.w_router, torch.zeros((-L.router.experts) % 4, cfg.width, dtype=dtype, device=self.device)], 0)
+                if gate_w is not None:                 # columns [2W, 2W + experts)
                     gate_b = torch.cat([gate_b, torch.zeros(rw.shape[0], dtype=dtype, device=self.device)], 0).contiguous()
+                    rw = torch.cat([gate_w, rw], 0)
+                gate_w = rw.contiguous()
             n2 = norm_w(p + "norm2") if mlp is not None and not cfg.shared_norm else None
-            if gate_w is not None and cfg.shared_norm and isinstance(mixer, (LatentAttention, Retention)):
+            if gate_w is not None and cfg.shared_norm and isinstance(mixer, (LatentAttention, Retention, PagedChunkAttention)) and mixer.b_in is None:
                 # every projection of the layer's one normed input in ONE linear: [mixer inputs (padded to 4 columns) | gates | router]
                 pad = (-mixer.w_in.shape[0]) % 4
                 zrow = torch.zeros(pad, cfg.width, dtype=dtype, device=self.device)
                 self.n_mix[i] = (mixer.w_in.shape[0], mixer.w_in.shape[0] + pad)
-                gate_b = torch.cat([torch.zeros(mixer.w_in.shape[0] + pad, dtype=dtype, device=self.device), gate_b], 0).contiguous()
+                if gate_b is not None:
+                    gate_b = torch.cat([torch.zeros(mixer.w_in.shape[0] + pad, dtype=dtype, device=self.device), gate_b], 0).contiguous()
                 gate_w = torch.cat([mixer.w_in, zrow, gate_w], 0).contiguous()
                 mixer.w_in = None                      # lives on as the leading rows of the shared weight
             self.layers.append((L, mixer, mlp, norm_w(p + "norm1"), n2, gate_w, gate_b))
         self.runs = cfg.layer_runs()
         if cfg.loop is not None and (cfg.depth_mix or cfg.out_norm or any(getattr(L.mixer, "kv_from", None) is not None for L in cfg.layers)):
             raise NotImplementedError("a loop over layers is not combined with depth averages, normed outputs or shared keys and values")
+        self.pass_at, self.loop_in, self.loop_step = {}, None, None
+        if cfg.loop_input:
+            if cfg.sequential:
+                raise NotImplementedError("a loop fed with the embedding output is built for parallel layers")
+            self.pass_at = cfg.pass_starts()
+            self.loop_in, self.loop_step = get("loop.in"), get("loop.step")
+            if self.loop_in.shape != (cfg.width, 2 * cfg.width) or self.loop_step.shape != (cfg.loop[2], cfg.width):
+                raise ValueError(f"loop.in {tuple(self.loop_in.shape)} / loop.step {tuple(self.loop_step.shape)} for {cfg.loop[2]} passes of width {cfg.width}")
         self.stream_mix = []                             # per layer: (in, out, mix) of both sublayers, fp32 on the device (no second entry without an MLP)
         if cfg.streams:
             if not cfg.sequential or cfg.depth_mix or cfg.out_norm or cfg.bigram is not None or cfg.embed_scale != 1.0:
@@ -491,19 +555,37 @@ class HybridModel:
             return self._forward_out_norm(batch, caches, collect)
         if cfg.sequential:
             return self._forward_sequential(batch, caches, collect)
-        x = hops.embed(batch.tokens, self.embed)
+        T, W = batch.tokens.numel(), cfg.width
+        pair = None                                    # [stream | embedding output] rounded: the operand of the linear in front of every pass of a loop
+        if self.pass_at:
+            pair = torch.empty(T, 2 * W, dtype=self.dtype, device=self.device)
+            x, _ = hops.embed_scaled(batch.tokens, self.embed, cfg.embed_scale, copy=pair[:, W:])
+        elif cfg.embed_scale != 1.0:
+            x, _ = hops.embed_scaled(batch.tokens, self.embed, cfg.embed_scale)
+        else:
+            x = hops.embed(batch.tokens, self.embed)
         a = b = g = None
         shared = self.n_mix
-        for i, cache in zip(self.runs, caches):
+        router_at = 2 * W if cfg.branch_gates else 0   # column of the router's logits behind the mixer's
+        for run, (i, cache) in enumerate(zip(self.runs, caches)):
             L, mixer, mlp, n1, n2, gate_w, gate_b = self.layers[i]
-            h1, h2 = hops.residual_norm(x, a, b, cfg.residual_mult, n1, n2, cfg.eps, weight_offset=cfg.norm_offset, gate=g)
-            if collect is not None and a is not None:
+            bg = g if cfg.branch_gates else None
+            done = collect is not None and a is not None
+            if run in self.pass_at:                    # x <- A [x; x0] + s: the last layer's branches join the stream in the launch that rounds it
+                hops.residual_round(x, a, b, cfg.residual_mult, pair[:, :W], gate=bg)
+                if done:
+                    collect.append(x.clone())
+                x = hops.dense_linear(pair, self.loop_in, self.loop_step[self.pass_at[run]], out_dtype=torch.float32)
+                a = b = bg = None
+                done = False
+            h1, h2 = hops.residual_norm(x, a, b, cfg.residual_mult, n1, n2, cfg.eps, weight_offset=cfg.norm_offset, gate=bg)
+            if done:
                 collect.append(x.clone())
             if cfg.shared_norm:
                 h2 = h1
-            if i in shared:                            # the mixer's projections are the leading rows of the gates' weight
+            if i in shared:                            # the mixer's projections are the leading rows of the shared weight
                 n_in, n_pad = shared[i]
-                if h1.shape[0] <= 16:                  # decode-sized steps: one launch streams the whole weight
+                if T <= 16 or not cfg.branch_gates:    # decode-sized steps, and a few columns behind the mixer's: one launch streams the whole weight
                     g = hops.dense_linear(h1, gate_w, gate_b, out_dtype=torch.float32)
                     proj, g = g[:, :n_in], g[:, n_pad:]
                 else:                                  # prompt portions: the tile kernel is faster on the two halves (measured: 0.6 ms of a 2048-token prefill)
@@ -515,15 +597,16 @@ class HybridModel:
                 a = mixer.forward(h1, batch, *cache) if isinstance(cache, tuple) else mixer.forward(h1, batch, cache)
             if mlp is None:
                 b = None
-            elif g is not None and isinstance(mlp, RoutedExperts):
-                b = mlp.forward(h2, g[:, 2 * cfg.width: 2 * cfg.width + L.router.experts], defer=True)   # summed by the next residual kernel
+            elif isinstance(mlp, RoutedExperts):       # summed by the next residual kernel
+                b = mlp.forward(h2, g[:, router_at: router_at + L.router.experts] if g is not None else None, defer=True)
             else:
                 b = mlp.forward(h2)
+        bg = g if cfg.branch_gates else None
         if collect is not None:
-            hops.residual_norm(x, a, b, cfg.residual_mult, self.final_norm, None, cfg.eps, weight_offset=cfg.norm_offset, gate=g)
+            hops.residual_norm(x, a, b, cfg.residual_mult, self.final_norm, None, cfg.eps, weight_offset=cfg.norm_offset, gate=bg)
             collect.append(x.clone())
-            a = b = g = None
-        hf, _ = hops.residual_norm(x, a, b, cfg.residual_mult, self.final_norm, None, cfg.eps, weight_offset=cfg.norm_offset, rows=batch.want, gate=g)
+            a = b = bg = None
+        hf, _ = hops.residual_norm(x, a, b, cfg.residual_mult, self.final_norm, None, cfg.eps, weight_offset=cfg.norm_offset, rows=batch.want, gate=bg)
         return hops.dense_linear(hf, self.head, out_dtype=torch.float32, softcap=cfg.logit_softcap)
 
 

@@ -117,16 +117,23 @@ def embed(ids: torch.Tensor, table: torch.Tensor, *, prev: Optional[torch.Tensor
     return out
 
 
-def embed_scaled(ids: torch.Tensor, table: torch.Tensor, scale: float, *, rounded: bool = False):
+def embed_scaled(ids: torch.Tensor, table: torch.Tensor, scale: float, *, rounded: bool = False, copy: Optional[torch.Tensor] = None):
     """(fp32 stream rows [T, W] = table[ids] * scale, the same rows in the table's dtype or None): `rounded` asks for the second tensor, the input
-    of the first sublayer of a stack whose sublayers read the stream itself."""
+    of the first sublayer of a stack whose sublayers read the stream itself.  copy: a [T, W] tensor (columns of a wider buffer are fine) that the
+    rounded rows are written to."""
     _dev(ids, torch.int32, "embed_scaled.ids")
     T, W = ids.numel(), table.shape[1]
     out = torch.empty(T, W, dtype=torch.float32, device=table.device)
-    outh = torch.empty(T, W, dtype=table.dtype, device=table.device) if rounded else None
+    outh = torch.empty(T, W, dtype=table.dtype, device=table.device) if rounded and copy is None else copy
+    ldh = W
+    if copy is not None:
+        _dev(copy, table.dtype, "embed_scaled.copy")
+        ldh = _rows(copy, "embed_scaled.copy")
+        if copy.shape != (T, W):
+            raise _C.Mi355Error(f"embed_scaled: copy {tuple(copy.shape)} for [{T}, {W}]")
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_embed_scaled(ids.data_ptr(), T, table.data_ptr(), W, table.shape[0], float(scale), out.data_ptr(), _p(outh),
-                                                              act_code(table.dtype), _stream()), "hy_embed_scaled")
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_embed_scaled_ex(ids.data_ptr(), T, table.data_ptr(), W, table.shape[0], float(scale), out.data_ptr(), _p(outh), ldh,
+                                                                 act_code(table.dtype), _stream()), "hy_embed_scaled")
     return out, outh
 
 
@@ -267,36 +274,44 @@ def streams(X: torch.Tensor, *, mix: Optional[torch.Tensor] = None, write: Optio
     return h
 
 
+def _residual_branches(x: torch.Tensor, a: Optional[torch.Tensor], b, gate: Optional[torch.Tensor], name: str):
+    """Checks of a residual update's operands -> (the plain second branch, the MoeSum or None, the gate's row stride)."""
+    _dev(x, torch.float32, name + ".x")
+    W, ms = x.shape[1], None
+    if isinstance(b, MoeSum):                 # b: a tensor, or the parts of a mixture's sum
+        ms, b = b, b.extra
+        _dev(ms.y, torch.float32, name + ".moe.y"); _dev(ms.wts, torch.float32, name + ".moe.wts"); _dev(ms.place_of, torch.int32, name + ".moe.place")
+        if ms.wts.shape[0] != x.shape[0] or ms.y.shape != (ms.wts.numel(), W) or ms.place_of.numel() != ms.wts.numel() or not (ms.y.is_contiguous() and ms.wts.is_contiguous()):
+            raise _C.Mi355Error(f"{name}: mixture sum y {tuple(ms.y.shape)} wts {tuple(ms.wts.shape)} against the stream {tuple(x.shape)}")
+    for t, nm in ((a, ".a"), (b, ".b")):
+        if t is not None:
+            _dev(t, torch.float32, name + nm)
+            if t.shape != x.shape or not t.is_contiguous():
+                raise _C.Mi355Error(f"{name}{nm}: {tuple(t.shape)} against the stream {tuple(x.shape)}")
+    ldg = 0
+    if gate is not None:
+        _dev(gate, torch.float32, name + ".gate")
+        ldg = _rows(gate, name + ".gate")
+        if gate.shape[0] != x.shape[0] or gate.shape[1] < 2 * W:
+            raise _C.Mi355Error(f"{name}.gate: {tuple(gate.shape)} for two gates of the stream {tuple(x.shape)}")
+    if not x.is_contiguous():
+        raise _C.Mi355Error(f"{name}: the stream must be contiguous")
+    return b, ms, ldg
+
+
 def residual_norm(x: torch.Tensor, a: Optional[torch.Tensor], b, mult: float, w1: torch.Tensor,
                   w2: Optional[torch.Tensor], eps: float, *, weight_offset: float = 0.0, rows: Optional[torch.Tensor] = None,
                   gate: Optional[torch.Tensor] = None):
     """x <- x + mult * (a + b) on the fp32 stream (in place; skipped for absent branches, and x is only read when `rows` gathers), then
     RMS norms of the new rows under w1 and w2 (stored weight + weight_offset).  -> (h1, h2) in the weights' dtype.
     gate: fp32 [T, >= 2 W] pre-activations; a is multiplied by sigmoid(gate[:, :W]) and b by sigmoid(gate[:, W:2W]) before they are added."""
-    _dev(x, torch.float32, "residual_norm.x")
+    b, ms, ldg = _residual_branches(x, a, b, gate, "residual_norm")
     W = x.shape[1]
     n = x.shape[0] if rows is None else rows.numel()
-    ms = None
-    if isinstance(b, MoeSum):                 # b: a tensor, or the parts of a mixture's sum
-        ms, b = b, b.extra
-        _dev(ms.y, torch.float32, "residual_norm.moe.y"); _dev(ms.wts, torch.float32, "residual_norm.moe.wts"); _dev(ms.place_of, torch.int32, "residual_norm.moe.place")
-        if ms.wts.shape[0] != x.shape[0] or ms.y.shape != (ms.wts.numel(), W) or ms.place_of.numel() != ms.wts.numel() or not (ms.y.is_contiguous() and ms.wts.is_contiguous()):
-            raise _C.Mi355Error(f"residual_norm: mixture sum y {tuple(ms.y.shape)} wts {tuple(ms.wts.shape)} against the stream {tuple(x.shape)}")
-    for t, nm in ((a, "a"), (b, "b")):
-        if t is not None:
-            _dev(t, torch.float32, "residual_norm." + nm)
-            if t.shape != x.shape or not t.is_contiguous():
-                raise _C.Mi355Error(f"residual_norm.{nm}: {tuple(t.shape)} against the stream {tuple(x.shape)}")
     if rows is not None:
         _dev(rows, torch.int32, "residual_norm.rows")
-    ldg = 0
-    if gate is not None:
-        _dev(gate, torch.float32, "residual_norm.gate")
-        ldg = _rows(gate, "residual_norm.gate")
-        if gate.shape[0] != x.shape[0] or gate.shape[1] < 2 * W:
-            raise _C.Mi355Error(f"residual_norm.gate: {tuple(gate.shape)} for two gates of the stream {tuple(x.shape)}")
-    if not x.is_contiguous() or w1.numel() != W or (w2 is not None and (w2.numel() != W or w2.dtype != w1.dtype)):
-        raise _C.Mi355Error("residual_norm: stream must be contiguous and the weights [W] of one dtype")
+    if w1.numel() != W or (w2 is not None and (w2.numel() != W or w2.dtype != w1.dtype)):
+        raise _C.Mi355Error("residual_norm: the weights must be [W] of one dtype")
     h1 = torch.empty(n, W, dtype=w1.dtype, device=x.device)
     h2 = torch.empty(n, W, dtype=w1.dtype, device=x.device) if w2 is not None else None
     if n:
@@ -305,6 +320,22 @@ def residual_norm(x: torch.Tensor, a: Optional[torch.Tensor], b, mult: float, w1
                                                                      _p(ms.y) if ms else None, _p(ms.place_of) if ms else None, _p(ms.wts) if ms else None,
                                                                      ms.wts.shape[1] if ms else 0, act_code(w1.dtype), _stream()), "hy_residual_norm")
     return h1, h2
+
+
+def residual_round(x: torch.Tensor, a: Optional[torch.Tensor], b, mult: float, raw: torch.Tensor, *, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The update of residual_norm without a norm: x <- x + mult * (a + b) in place, and the new rows rounded to raw's dtype in raw [T, W] (columns of a
+    wider buffer are fine): the operand of a linear that reads the stream itself."""
+    b, ms, ldg = _residual_branches(x, a, b, gate, "residual_round")
+    _dev(raw, raw.dtype, "residual_round.raw")
+    ldraw = _rows(raw, "residual_round.raw")
+    if raw.shape != x.shape:
+        raise _C.Mi355Error(f"residual_round: raw {tuple(raw.shape)} for the stream {tuple(x.shape)}")
+    T, W = x.shape
+    if T:
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_residual_round(x.data_ptr(), _p(a), _p(b), _p(gate), ldg, float(mult), T, W, raw.data_ptr(), ldraw,
+                                                                _p(ms.y) if ms else None, _p(ms.place_of) if ms else None, _p(ms.wts) if ms else None,
+                                                                ms.wts.shape[1] if ms else 0, act_code(raw.dtype), _stream()), "hy_residual_round")
+    return raw
 
 
 def attn_geometry(heads, kv_heads, dim, vdim, rot_dims, rot_layout, v_layout, page, max_blocks, num_pages, v_ld=0):
@@ -357,11 +388,11 @@ def _ogate(gate: Optional[torch.Tensor], T: int, heads: int, vdim: int, name: st
 
 
 def attn_rows(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[torch.Tensor], vfreq, pos, seq, block_table, kcache, vcache,
-              heads: int, vdim: int, *, window: int = 0, softcap: float = 0.0, out_gate: Optional[torch.Tensor] = None):
+              heads: int, vdim: int, *, window: int = 0, softcap: float = 0.0, out_gate: Optional[torch.Tensor] = None, keep: int = 0):
     """Attention of every row over its sequence's pages -> [T, heads * vdim] in the cache dtype.  sink: fp32 [heads] or None; exp(sink[h])
     joins head h's softmax denominator.  Few rows over long block tables (decode steps) are dealt over several blocks per (row, head) whose
     partial sums a second launch merges; the count depends on the rows and the table's width only.  window > 0: a row at position i sees
-    the keys j with 0 <= i - j < window; softcap > 0: cap * tanh(score / cap) on the scaled scores; out_gate fp32 [T, heads] or [T, heads * vdim]
+    the keys j with 0 <= i - j < window, and with keep > 0 also the keys j < keep (j <= i); softcap > 0: cap * tanh(score / cap) on the scaled scores; out_gate fp32 [T, heads] or [T, heads * vdim]
     (a column slice is fine): head h of a row, or every channel of it, is multiplied by the sigmoid of its entry."""
     _dev(q, torch.float32, "attn_rows.q")
     T = q.shape[0]
@@ -371,14 +402,14 @@ def attn_rows(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[to
     if chunk == 0 and T * heads <= 2048:                   # sixteen waves per block: one 64-key tile per wave and block where the chip has room
         tiles = (block_table.shape[1] * geom[7] + 63) // 64
         if window > 0:
-            tiles = min(tiles, (window + 63) // 64 + 1)
+            tiles = min(tiles, (window + keep + 63) // 64 + 1)
         splits = max(1, min(16, (tiles + 15) // 16, 1024 // (T * heads)))
         if splits > 1:
             parts = torch.empty(T * heads * splits * (vdim + 2), dtype=torch.float32, device=q.device)
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_rows_ex2(q.data_ptr(), _rows(q, "attn_rows.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_rows_ex3(q.data_ptr(), _rows(q, "attn_rows.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
                                                               pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), T, kcache.data_ptr(), vcache.data_ptr(),
-                                                              out.data_ptr(), splits, _p(parts), int(window), float(softcap), gp, ldg, gch, act_code(kcache.dtype),
+                                                              out.data_ptr(), splits, _p(parts), int(window), int(keep), float(softcap), gp, ldg, gch, act_code(kcache.dtype),
                                                               _stream()), "hy_attn_rows")
     return out
 
@@ -389,7 +420,7 @@ def attn_tiles_supported(dtype: torch.dtype, dim: int, vdim: int, value_rot: boo
 
 
 def attn_tiles(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[torch.Tensor], vfreq, pos, seq, block_table, tile_row0, tile_n, kcache, vcache,
-               heads: int, vdim: int, *, window: int = 0, softcap: float = 0.0, out_gate: Optional[torch.Tensor] = None):
+               heads: int, vdim: int, *, window: int = 0, softcap: float = 0.0, out_gate: Optional[torch.Tensor] = None, keep: int = 0):
     """attn_rows for prompt portions on the matrix cores: tile t = rows tile_row0[t] .. + tile_n[t] - 1 (at most 16 consecutive rows of one
     sequence); every row of the batch must lie in exactly one tile."""
     _dev(q, torch.float32, "attn_tiles.q"); _dev(tile_row0, torch.int32, "attn_tiles.tile_row0"); _dev(tile_n, torch.int32, "attn_tiles.tile_n")
@@ -397,9 +428,9 @@ def attn_tiles(q: torch.Tensor, scale: float, geom, chunk: int, sink: Optional[t
     out = torch.empty(T, heads * vdim, dtype=kcache.dtype, device=q.device)
     gp, ldg, gch = _ogate(out_gate, T, heads, vdim, "attn_tiles.out_gate")
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_tiles_ex2(q.data_ptr(), _rows(q, "attn_tiles.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_attn_tiles_ex3(q.data_ptr(), _rows(q, "attn_tiles.q"), float(scale), geom, int(chunk), _sink(sink, heads), _p(vfreq),
                                                                pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), tile_row0.data_ptr(), tile_n.data_ptr(),
-                                                               tile_row0.numel(), kcache.data_ptr(), vcache.data_ptr(), out.data_ptr(), int(window),
+                                                               tile_row0.numel(), kcache.data_ptr(), vcache.data_ptr(), out.data_ptr(), int(window), int(keep),
                                                                float(softcap), gp, ldg, gch, act_code(kcache.dtype), _stream()), "hy_attn_tiles")
     return out
 
@@ -611,8 +642,11 @@ def head_norm(o: torch.Tensor, heads: int, vdim: int, w: Optional[torch.Tensor],
               out_dtype: Optional[torch.dtype] = None, gate_act: str = "silu", den: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per-head RMS norm of o (fp32 [T, heads * vdim]) under the weight w ([vdim] shared by the heads, or [heads * vdim]; None: unit RMS only,
     output in `out_dtype`), times gate_act(gate[:, goff:]) ("silu" or "sigmoid") when a gate is given.  den (fp32 [T, heads]): every head is divided
-    by its entry before the norm."""
+    by its entry before the norm.  o may be columns of a wider buffer."""
     _dev(o, torch.float32, "head_norm.o")
+    ldo = _rows(o, "head_norm.o")
+    if o.shape[1] != heads * vdim:
+        raise _C.Mi355Error(f"head_norm: o {tuple(o.shape)} for {heads} heads of {vdim}")
     T = o.shape[0]
     dt = w.dtype if w is not None else out_dtype
     out = torch.empty(T, heads * vdim, dtype=dt, device=o.device)
@@ -628,7 +662,7 @@ def head_norm(o: torch.Tensor, heads: int, vdim: int, w: Optional[torch.Tensor],
             _dev(den, torch.float32, "head_norm.den")
             if den.shape != (T, heads) or not den.is_contiguous():
                 raise _C.Mi355Error(f"head_norm: denominators {tuple(den.shape)} for {T} rows of {heads} heads")
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_head_norm_ex2(o.data_ptr(), T, heads, vdim, _p(w), float(eps), _p(gate),
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_head_norm_ex3(o.data_ptr(), ldo, T, heads, vdim, _p(w), float(eps), _p(gate),
                                                               0 if gate is None else _rows(gate, "head_norm.gate"), goff, out.data_ptr(), per_head,
                                                               1 if gate_act == "sigmoid" else 0, _p(den), act_code(dt), _stream()), "hy_head_norm")
     return out
@@ -689,22 +723,30 @@ def latent_geometry(heads, dim, rot_dim, rank, padded, rot_span, page, max_block
 
 
 def latent_prep(proj: torch.Tensor, doff: int, geom, freq, mag: float, cw: torch.Tensor, eps: float, pos, seq, block_table, qn: torch.Tensor,
-                qabs: torch.Tensor, cache: torch.Tensor):
+                qabs: torch.Tensor, cache: torch.Tensor, *, q: Optional[torch.Tensor] = None, layout: int = 0):
     """Latent attention, before the scores: from the fp32 projections [T, ld] (query heads from column 0, down projection from column doff) write
     the token's cached row [normed latent | turned shared key part | zeros], the un-rotated query parts (qn, activation dtype) and the turned
-    query parts + padding into columns rank.. of every head's absorbed query row (qabs fp32)."""
+    query parts + padding into columns rank.. of every head's absorbed query row (qabs fp32).  q: the query heads as an fp32 tensor of their own (proj
+    then only holds the down projection at doff); layout: pairs of the rotation (LAYOUTS)."""
     _dev(proj, torch.float32, "latent_prep.proj"); _dev(qabs, torch.float32, "latent_prep.qabs")
     _dev(qn, cache.dtype, "latent_prep.qn"); _dev(cw, cache.dtype, "latent_prep.norm")
-    T = proj.shape[0]
+    T, ld = proj.shape[0], _rows(proj, "latent_prep.proj")
     H, dim, dr, R, dpad = geom[0], geom[1], geom[2], geom[3], geom[4]
     if qn.shape != (T, H * dim) or qabs.shape != (T, H * dpad) or not qn.is_contiguous() or not qabs.is_contiguous() or cw.numel() != R:
         raise _C.Mi355Error(f"latent_prep: qn {tuple(qn.shape)} qabs {tuple(qabs.shape)} norm {tuple(cw.shape)}")
     if cache.dim() != 3 or cache.shape[1:] != (geom[6], dpad) or cache.shape[0] != geom[8] or not cache.is_contiguous():
         raise _C.Mi355Error(f"latent_prep: cache {tuple(cache.shape)} against pages of {geom[6]} rows of {dpad}")
+    if q is not None:
+        _dev(q, torch.float32, "latent_prep.q")
+    elif doff < H * (dim + dr):
+        raise _C.Mi355Error(f"latent_prep: down projection at column {doff} behind {H} heads of {dim + dr}")
+    src = proj if q is None else q
+    if src.shape[0] != T or src.shape[1] < H * (dim + dr) or proj.shape[1] < doff + R + dr:
+        raise _C.Mi355Error(f"latent_prep: queries {tuple(src.shape)} / projections {tuple(proj.shape)} (down projection at {doff}) for {H} heads of {dim} + {dr}, rank {R}")
     if T:
-        _C.check_hybrid(_C.hybrid_lib().mi355_hy_latent_prep(proj.data_ptr(), _rows(proj, "latent_prep.proj"), doff, geom, _p(freq), float(mag), cw.data_ptr(),
-                                                             float(eps), pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), T, qn.data_ptr(),
-                                                             qabs.data_ptr(), cache.data_ptr(), act_code(cache.dtype), _stream()), "hy_latent_prep")
+        _C.check_hybrid(_C.hybrid_lib().mi355_hy_latent_prep_ex(src.data_ptr(), _rows(src, "latent_prep.q"), proj.data_ptr() + 4 * doff, ld, geom, int(layout), _p(freq),
+                                                                float(mag), cw.data_ptr(), float(eps), pos.data_ptr(), seq.data_ptr(), block_table.data_ptr(), T,
+                                                                qn.data_ptr(), qabs.data_ptr(), cache.data_ptr(), act_code(cache.dtype), _stream()), "hy_latent_prep")
 
 
 def rotary(buf: torch.Tensor, segments, rot_dims: int, layout: int, freq: torch.Tensor, mag: float, pos: torch.Tensor):

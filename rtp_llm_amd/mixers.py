@@ -5,7 +5,7 @@
     optional unit-normed values and optional value rotation (values are turned by their own position when cached and the head output
     is turned back by the query's position, so a value enters the sum turned by the distance).  A layer may read the cache that an
     earlier layer with the same geometry wrote (`kv_from`) and then has no key / value projections.  Further options, each off by default:
-    a sliding window instead of the block mask, a tanh cap on the scaled scores, a temperature on the queries that grows with the
+    a sliding window (which may keep the first tokens of the sequence) instead of the block mask, a tanh cap on the scaled scores, a temperature on the queries that grows with the
     logarithm of the position, RMS-normed queries and keys under weights shared by the heads, YaRN-scaled rotary steps, biases on the
     projections, and a sigmoid gate per head on the output.
   * ``GeneralizedDeltaRule`` -- S_t = diag(w_t) S_(t-1) - (a_t * u_t)(u_t^T S_(t-1)) + k_t v_t^T, o_t = S_t^T r_t per head with the state in an
@@ -18,7 +18,8 @@
   * ``LatentAttention`` -- attention whose keys and values are linear images of ONE low-rank latent vector per token, plus a rotated key
     part shared by all heads.  Only the normed latent and that key part are cached (one row per token for all heads); the key
     up-projection is moved to the query side and the value up-projection behind the weighted sum, so the paged kernels see multi-query
-    attention over the cached rows.  Rotary with optional YaRN frequency scaling, a learned per-head softmax sink, a sigmoid output gate.
+    attention over the cached rows.  Queries come from the input or from a normed latent of their own.  Rotary of either pair layout with optional
+    YaRN frequency scaling, a learned per-head softmax sink, a sigmoid output gate per channel or per head.
   * ``Retention`` -- the same recurrence with one constant decay per head, rotated q and k, unit-RMS heads and a silu output gate.
   * ``LightningAttention`` -- that recurrence with silu on q, k and v, one RMS norm over all heads together and a sigmoid output gate.
   * ``ChannelDelta`` -- the gated delta rule with a decay per key channel, S <- diag(g) S, S <- S + beta k (v - S^T k)^T, o = S^T q, on unit queries and
@@ -100,6 +101,7 @@ class AttentionSpec:
     value_layout: str = "interleaved"
     kv_from: Optional[int] = None
     window: int = 0                      # > 0 (chunk must be 0): position i sees the keys j with 0 <= i - j < window
+    keep_first: int = 0                  # with a window: the first keep_first positions of the sequence stay visible to everything behind them
     softcap: float = 0.0                 # > 0: scaled scores become softcap * tanh(score / softcap)
     q_temp: Optional[tuple] = None       # (coef, every): queries at position p are multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)
     qk_norm: bool = False                # queries and keys are RMS-normed per head under weights [dim] shared by the heads, before the rotation
@@ -189,6 +191,8 @@ class PagedChunkAttention:
             raise ValueError(f"attention: {s.heads} query heads over {s.kv_heads} key/value heads")
         if s.window and s.chunk:
             raise ValueError("attention: a sliding window and a block mask exclude each other")
+        if s.window < 0 or s.keep_first < 0:
+            raise ValueError(f"attention: window {s.window}, {s.keep_first} kept tokens")
         self.owns_cache = s.kv_from is None
         self.n_gate = 0 if not s.out_gate else s.heads * (s.vdim if s.gate_channels else 1)
         if s.out_gate and weights["g"].shape[0] != self.n_gate:
@@ -250,7 +254,7 @@ class PagedChunkAttention:
                        kcache if write else None, vcache if write else None, q_norm=self.q_norm, k_norm=self.k_norm, mag=self.mag, q_temp=s.q_temp,
                        cache_dtype=kcache.dtype, norm_whole=s.qk_norm_whole)
         T = qkv.shape[0]
-        extra = dict(window=s.window, softcap=s.softcap, out_gate=qkv[:, self.goff:self.goff + self.n_gate] if s.out_gate else None)
+        extra = dict(window=s.window, keep=s.keep_first, softcap=s.softcap, out_gate=qkv[:, self.goff:self.goff + self.n_gate] if s.out_gate else None)
         # prompt portions (tiles mostly full) go to the matrix-core kernel, decode rows to the one that spreads a row's keys over four waves
         if (self.use_tiles and batch.tile_row0 is not None and batch.tile_row0.numel() * 4 <= T
                 and hops.attn_tiles_supported(kcache.dtype, s.dim, s.vdim, self.vfreq is not None, hops.LAYOUTS[s.value_layout])):
@@ -343,24 +347,38 @@ class LatentAttentionSpec:
     scale: float
     rot: Optional[RotarySpec] = None     # turns the first rot.dims of the rot_dim channels
     sink: bool = True                    # learned per-head sink logit in the softmax denominator
-    out_gate: bool = True                # heads multiplied by sigmoid(W_g h) before the output projection
+    out_gate: bool = True                # heads multiplied by sigmoid(W_g h) before the output projection ...
+    gate_channels: bool = True           # ... one number per head and value channel, or one per head
+    query_latent: bool = False           # queries are W_uq N(W_dq h), N an RMS norm with a weight per channel, instead of W_q h
 
 
 class LatentAttention:
-    """weights: q [H (dim + rot_dim), W], dkv [kv_rank + rot_dim, W], dkv.norm [kv_rank], uk [H dim, kv_rank], uv [H vdim, kv_rank], sink [H],
-    g [H vdim, W], o [W, H vdim].  Cached per token: [normed latent | turned shared key part | zeros] in `padded` channels (a multiple of 32,
-    so that the matrix-core attention takes the rows); the values are the first kv_rank channels of the same row."""
+    """weights: q [H (dim + rot_dim), W] (or dq [q_rank, W], dq.norm [q_rank], uq [H (dim + rot_dim), q_rank]), dkv [kv_rank + rot_dim, W], dkv.norm [kv_rank],
+    uk [H dim, kv_rank], uv [H vdim, kv_rank], sink [H], g [H vdim, W] or [H, W], o [W, H vdim].  Cached per token: [normed latent | turned shared key part |
+    zeros] in `padded` channels (a multiple of 32, so that the matrix-core attention takes the rows); the values are the first kv_rank channels of the
+    same row.  A gate per head is applied to the weighted latent (the value up-projection behind it is linear), a gate per channel behind that projection."""
 
     def __init__(self, spec: LatentAttentionSpec, weights: Dict[str, torch.Tensor], eps: float, page: int, device):
         s = self.spec = spec
         self.eps, self.page = eps, page
         H, d, dr, R = s.heads, s.dim, s.rot_dim, s.kv_rank
         self.padded = -(-(R + dr) // 32) * 32
-        if s.rot is not None and (s.rot.dims > dr or s.rot.layout != "interleaved"):
-            raise ValueError(f"latent attention: rotary span {s.rot.dims} of {dr} channels ({s.rot.layout})")
-        parts = [weights["q"], weights["dkv"]] + ([weights["g"]] if s.out_gate else [])
+        if s.rot is not None and s.rot.dims > dr:
+            raise ValueError(f"latent attention: rotary span {s.rot.dims} of {dr} channels")
+        self.n_gate = 0 if not s.out_gate else H * (s.vdim if s.gate_channels else 1)
+        for n, rows in (("uq" if s.query_latent else "q", H * (d + dr)), ("dkv", R + dr), ("uk", H * d), ("uv", H * s.vdim)) + ((("g", self.n_gate),) if s.out_gate else ()):
+            if weights[n].shape[0] != rows:
+                raise ValueError(f"latent attention: weight {n} {tuple(weights[n].shape)} for {H} heads of {d} + {dr} and {s.vdim}, rank {R}")
+        parts = [weights["dq" if s.query_latent else "q"], weights["dkv"]] + ([weights["g"]] if s.out_gate else [])
         self.w_in = torch.cat(parts, 0).contiguous()
-        self.doff, self.goff = H * (d + dr), H * (d + dr) + R + dr
+        self.b_in = None
+        self.doff = parts[0].shape[0]                    # columns of the input linear: queries (or their latent) | down projection | gate
+        self.goff = self.doff + R + dr
+        self.w_uq = self.q_norm = None
+        if s.query_latent:
+            self.w_uq, self.q_norm = weights["uq"].contiguous(), weights["dq.norm"].contiguous()
+            if self.w_uq.shape[1] != self.doff or self.q_norm.numel() != self.doff:
+                raise ValueError(f"latent attention: query latent of {self.doff}, norm {tuple(self.q_norm.shape)}, up-projection {tuple(self.w_uq.shape)}")
         self.c_norm = weights["dkv.norm"].contiguous()
         # key up-projection on the query side: per head [kv_rank, dim] (q_abs = W_uk,h^T q_h); value up-projection per head [vdim, kv_rank]
         self.w_uk_t = weights["uk"].view(H, d, R).transpose(1, 2).contiguous()
@@ -394,16 +412,23 @@ class LatentAttention:
             proj = hops.dense_linear(h, self.w_in, out_dtype=torch.float32)
         qn = torch.empty(T, H * s.dim, dtype=self.act, device=h.device)
         qabs = torch.empty(T, H * self.padded, dtype=torch.float32, device=h.device)
-        hops.latent_prep(proj, self.doff, lgeom, self.freq, self.mag, self.c_norm, self.eps, batch.pos, batch.seq, batch.block_table, qn, qabs, cache)
+        q = None
+        if s.query_latent:
+            q = hops.dense_linear(hops.head_norm(proj[:, :self.doff], 1, self.doff, self.q_norm, self.eps), self.w_uq, out_dtype=torch.float32)
+        hops.latent_prep(proj, self.doff, lgeom, self.freq, self.mag, self.c_norm, self.eps, batch.pos, batch.seq, batch.block_table, qn, qabs, cache, q=q,
+                         layout=hops.LAYOUTS[s.rot.layout] if s.rot is not None else 0)
         hops.dense_grouped(qn, self.w_uk_t, x_step=s.dim, y_step=self.padded, out_dtype=torch.float32, out=qabs)
         kc = cache.view(cache.shape[0], 1, self.page, self.padded)
+        gate = proj[:, self.goff:self.goff + self.n_gate] if s.out_gate else None
+        head_gate = gate if not s.gate_channels else None
         if (self.use_tiles and batch.tile_row0 is not None and batch.tile_row0.numel() * 4 <= T
                 and hops.attn_tiles_supported(cache.dtype, self.padded, R, False, 0)):
-            ol = hops.attn_tiles(qabs, s.scale, ageom, 0, self.sink, None, batch.pos, batch.seq, batch.block_table, batch.tile_row0, batch.tile_n, kc, kc, H, R)
+            ol = hops.attn_tiles(qabs, s.scale, ageom, 0, self.sink, None, batch.pos, batch.seq, batch.block_table, batch.tile_row0, batch.tile_n, kc, kc, H, R,
+                                 out_gate=head_gate)
         else:
-            ol = hops.attn_rows(qabs, s.scale, ageom, 0, self.sink, None, batch.pos, batch.seq, batch.block_table, kc, kc, H, R)
-        # value up-projection per head; the output gate sigmoid(W_g h) is applied in its epilogue
-        o = hops.dense_grouped(ol, self.w_uv, x_step=R, y_step=s.vdim, mul_sigmoid=proj[:, self.goff:self.goff + H * s.vdim] if s.out_gate else None)
+            ol = hops.attn_rows(qabs, s.scale, ageom, 0, self.sink, None, batch.pos, batch.seq, batch.block_table, kc, kc, H, R, out_gate=head_gate)
+        # value up-projection per head; an output gate per channel is applied in its epilogue
+        o = hops.dense_grouped(ol, self.w_uv, x_step=R, y_step=s.vdim, mul_sigmoid=gate if s.gate_channels else None)
         return hops.dense_linear(o, self.w_o, out_dtype=torch.float32)
 
 

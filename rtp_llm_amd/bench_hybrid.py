@@ -18,6 +18,10 @@ the like Pokepel kernels against their rooflines.
 delta rule with a decay per key channel, squared-relu experts) beside the Nudorax member at equal width, depth, heads, vocabulary and feed-forward work,
 and its kernels beside the like Nudorax kernels (the delta rule beside Nepudra's).
 
+`--hybrid-design kerotar` measures the Kerotar member (window attention that keeps the first tokens, latent attention with a query latent, parallel
+layers under one norm, a layer loop fed with the embedding output) beside the Pokepel member (latent attention, parallel layers under one norm, routed
+experts) at equal width, depth, heads and vocabulary, and its kernels beside the like Pokepel kernels (the windowed ones beside Nudorax's).
+
 Output: one JSON line {"hybrid_bench": {size: {"hybrid": {...}, "qwen2": {...}, "kernels": [...]}}} (with --hybrid-design pokepel:
 {"pokepel": {...}, "nufalorn": {...}, "kernels": [...]})."""
 import json
@@ -304,6 +308,55 @@ def dupenex_weights(cfg, dev, seed=0, rank=64):
     return w
 
 
+def kerotar_config(s, experts=16, top=4, window=1024, keep=64):
+    """Width, heads and vocabulary of `s`, as many layer RUNS as it has layers (two of the layers run twice, fed with the embedding output); grouped-query
+    attention over a window that keeps the first tokens, with a clamped gated MLP of the full FFN width, in every second layer; in the others latent
+    attention with Pokepel's sizes behind a query latent of half the width, with `experts` silu-gated experts of a quarter of the FFN width (`top` of them
+    per token: the dense MLP's work)."""
+    layers, hd = [], s["hd"]
+    for i in range(s["layers"] - 2):
+        if i % 2 == 0:
+            mx = {"heads": s["heads"], "kv_heads": s["kv"], "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": window, "keep_first": keep},
+                  "rot": {"base": 1e6, "dims": hd // 2}}
+            layers.append({"type": "attention", "mixer": mx, "mlp": {"kind": "dense", "ff": s["ff"], "limit": 7.0}})
+        else:
+            mx = {"heads": s["heads"], "dim": hd, "rot_dim": hd // 2, "vdim": hd, "kv_rank": 3 * hd // 2, "q_rank": s["width"] // 2, "scale": (hd + hd // 2) ** -0.5,
+                  "rot": {"base": 1e6, "dims": hd // 2}}
+            layers.append({"type": "latent_attention", "mixer": mx,
+                           "mlp": {"kind": "moe", "expert": {"ff": s["ff"] // 4 // 32 * 32}, "router": {"experts": experts, "top": top}}})
+    return {"architecture": "Kerotar", "layers": layers, "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0},
+            "loop": {"start": 2, "stop": 4, "times": 2}}
+
+
+def kerotar_weights(cfg, dev, seed=0):
+    g = torch.Generator(device=dev).manual_seed(seed)
+    W = cfg["width"]
+    lin = lambda o, i: (torch.randn(o, i, device=dev, generator=g) * i ** -0.5).bfloat16()
+    vec = lambda n, k=0.1, off=0.0: (torch.randn(n, device=dev, generator=g) * k + off).bfloat16()
+    w = {"embed": (torch.randn(cfg["vocab"], W, device=dev, generator=g) * 0.25).bfloat16(), "head": lin(cfg["vocab"], W), "final.norm": vec(W, 0.1, 1.0),
+         "loop.in": lin(W, 2 * W), "loop.step": (torch.randn(cfg["loop"]["times"], W, device=dev, generator=g) * 0.1).bfloat16()}
+    for i, L in enumerate(cfg["layers"]):
+        p, mx, mlp = f"l{i}.", L["mixer"], L["mlp"]
+        H, d, dv, q = mx["heads"], mx["dim"], mx["vdim"], f"l{i}.mix."
+        w[p + "norm1"] = vec(W, 0.1, 1.0)
+        if L["type"] == "attention":
+            G = mx["kv_heads"]
+            shapes = {"q": (H * d, W), "k": (G * d, W), "v": (G * dv, W), "o": (W, H * dv)}
+            w[q + "q.norm"], w[q + "k.norm"], w[q + "sink"] = vec(H * d, 0.1, 1.0), vec(G * d, 0.1, 1.0), vec(H, 1.0)
+        else:
+            dr, R, Rq = mx["rot_dim"], mx["kv_rank"], mx["q_rank"]
+            shapes = {"dq": (Rq, W), "uq": (H * (d + dr), Rq), "dkv": (R + dr, W), "uk": (H * d, R), "uv": (H * dv, R), "g": (H, W), "o": (W, H * dv)}
+            w[q + "dq.norm"], w[q + "dkv.norm"] = vec(Rq, 0.1, 1.0), vec(R, 0.1, 1.0)
+        for n, (o, k) in shapes.items():
+            w[q + n] = lin(o, k)
+        f = mlp["ff"] if mlp["kind"] == "dense" else mlp["expert"]["ff"]
+        if mlp["kind"] == "moe":
+            w[p + "mlp.router"] = lin(mlp["router"]["experts"], W)
+        for n in [""] if mlp["kind"] == "dense" else [f"e{j}." for j in range(mlp["router"]["experts"])]:
+            w[p + f"mlp.{n}gate"], w[p + f"mlp.{n}up"], w[p + f"mlp.{n}down"] = lin(f, W), lin(f, W), lin(W, f)
+    return w
+
+
 def timed(fn, reps=5, warm=2, graph=False):
     """Seconds per call.  graph: the calls are captured into one HIP graph and the replay is timed, so the figure is the kernels' own
     time and not the host's launch path (what a graph-replayed step pays)."""
@@ -339,7 +392,8 @@ def bench_hybrid_engine(s, dev, prompt, batch, steps, design="nufalorn"):
     from .hybrid import HybridConfig, HybridModel
     from .scheduler import ServingEngine
     make_cfg, make_w = {"pokepel": (pokepel_config, pokepel_weights), "nepudra": (nepudra_config, nepudra_weights),
-                        "nudorax": (nudorax_config, nudorax_weights), "dupenex": (dupenex_config, dupenex_weights)}.get(design, (hybrid_config, hybrid_weights))
+                        "nudorax": (nudorax_config, nudorax_weights), "dupenex": (dupenex_config, dupenex_weights),
+                        "kerotar": (kerotar_config, kerotar_weights)}.get(design, (hybrid_config, hybrid_weights))
     cfg = make_cfg(s)
     model = HybridModel(HybridConfig.from_json(cfg), make_w(cfg, dev), torch.bfloat16, dev)
     eng = ServingEngine(model, max_tokens=batch * (prompt + 8 * (steps + 3) + 128), max_seqs=batch, max_step_tokens=1 << 20)
@@ -1042,12 +1096,141 @@ def kernel_table_dupenex(s, dev, prompt):
     return rows
 
 
+def kernel_table_kerotar(s, dev, prompt):
+    """Kerotar's kernels at this size beside the like kernels of the Pokepel member (the windowed attention and the scaled embedding beside Nudorax's),
+    against max(bytes / HBM, flops / peak of the unit)."""
+    from . import hybrid_ops as hops
+    rows = []
+    timed_k = lambda fn: timed(fn, reps=10, warm=2, graph=True)
+    g = torch.Generator(device=dev).manual_seed(3)
+    bf = lambda *sh: torch.randn(*sh, device=dev, generator=g).bfloat16()
+    f32 = lambda *sh: torch.randn(*sh, device=dev, generator=g)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)
+    W, H, G, hd, ff = s["width"], s["heads"], s["kv"], s["hd"], s["ff"]
+    cfg, pcfg = kerotar_config(s), pokepel_config(s)
+    a, b = cfg["layers"][0]["mixer"], cfg["layers"][1]["mixer"]
+    moe, pmoe = cfg["layers"][1]["mlp"], next(L["mlp"] for L in pcfg["layers"] if L["mlp"]["kind"] == "moe")
+    window, keep, span = a["mask"]["size"], a["mask"]["keep_first"], a["rot"]["dims"]
+    R, dr, Rq = b["kv_rank"], b["rot_dim"], b["q_rank"]
+    fe, E, top, gr = moe["expert"]["ff"], moe["router"]["experts"], moe["router"]["top"], pmoe["router"]["groups"]
+    dpad = -(-(R + dr) // 32) * 32
+
+    def add(family, name, shape, t, nbytes, flops, peak):
+        roof = max(nbytes / HBM, flops / peak)
+        rows.append({"family": family, "kernel": name, "shape": shape, "us": round(t * 1e6, 1), "roofline_us": round(roof * 1e6, 2),
+                     "x_roofline": round(t / roof, 1)})
+
+    page = 64
+    nblk = (prompt + page - 1) // page + 1
+    bt = torch.arange(nblk, dtype=torch.int32, device=dev).reshape(1, nblk)
+    sink = f32(H)
+    geom = hops.attn_geometry(H, G, hd, hd, span, 1, 0, page, nblk, nblk)
+    ngeo = hops.attn_geometry(H, G, hd, hd, hd, 1, 0, page, nblk, nblk)
+    lgeo = hops.attn_geometry(H, 1, dpad, R, 0, 0, 0, page, nblk, nblk, v_ld=dpad)
+    kc, vc, lc = bf(nblk, G, page, hd), bf(nblk, G, page, hd), bf(nblk, 1, page, dpad)
+    for T_, name in ((prompt, "prefill"), (1, "decode")):
+        pos = torch.arange(T_, dtype=torch.int32, device=dev) if T_ > 1 else i32([prompt - 1])
+        seq = torch.zeros(T_, dtype=torch.int32, device=dev)
+        q, lq, gate = f32(T_, H * hd), f32(T_, H * dpad), f32(T_, H)
+        kw = float(sum(min(int(p) + 1, window) for p in pos.tolist()))
+        kk = float(sum(min(int(p) + 1, window + keep) for p in pos.tolist()))
+        kall = float(sum(int(p) + 1 for p in pos.tolist()))
+        byt = lambda keys: min(prompt, keys) * G * hd * 2 * 2 + T_ * H * hd * 6
+        shape, lshape = f"T={T_} H={H} G={G} hd={hd} ctx={prompt}", f"T={T_} H={H} row={dpad} rank={R} ctx={prompt}"
+        lb = prompt * dpad * 2 + T_ * H * (dpad * 4 + R * 2)
+        common = (pos, seq, bt)
+        if T_ > 1:
+            t0 = torch.arange(0, T_, 16, dtype=torch.int32, device=dev)
+            tn = torch.full_like(t0, 16)
+            run = lambda q_, ge, sk, k_, v_, vd, **kw_: timed_k(lambda: hops.attn_tiles(q_, 0.07, ge, 0, sk, None, *common, t0, tn, k_, v_, H, vd, **kw_))
+            kn, keys_b = "attn_tiles prefill", prompt
+        else:
+            run = lambda q_, ge, sk, k_, v_, vd, **kw_: timed_k(lambda: hops.attn_rows(q_, 0.07, ge, 0, sk, None, *common, k_, v_, H, vd, **kw_))
+            kn, keys_b = "attn_rows decode", window + keep
+        add("kerotar", f"{kn} (window {window} + {keep} kept, learned sinks)", shape, run(q, geom, sink, kc, vc, hd, window=window, keep=keep), byt(keys_b), 4.0 * kk * H * hd, MFMA_BF16)
+        add("nudorax", f"{kn} (window {window}, learned sinks)", shape, run(q, geom, sink, kc, vc, hd, window=window), byt(min(keys_b, prompt if T_ > 1 else window)), 4.0 * kw * H * hd, MFMA_BF16)
+        add("kerotar", f"{kn} latent (causal, head gates)", lshape, run(lq, lgeo, None, lc, lc, R, out_gate=gate), lb, 2.0 * kall * H * (dpad + R), MFMA_BF16)
+        add("pokepel", f"{kn} latent (causal, learned sinks)", lshape, run(lq, lgeo, sink, lc, lc, R), lb, 2.0 * kall * H * (dpad + R), MFMA_BF16)
+    freq = torch.ones(hd // 2, device=dev) * 1e-3
+    lg = hops.latent_geometry(H, hd, dr, R, dpad, dr, page, nblk, nblk)
+    hq = H * (hd + dr)
+    for T_ in (prompt, 8):
+        pos, seq = torch.arange(T_, dtype=torch.int32, device=dev), torch.zeros(T_, dtype=torch.int32, device=dev)
+        qkv, qw, kw_ = f32(T_, (H + 2 * G) * hd), bf(H * hd), bf(G * hd)
+        nb = T_ * ((H + 2 * G) * hd * 4 + H * hd * 4 + 2 * G * hd * 2)
+        for fam, nm, ge in (("kerotar", "half the head turned", geom), ("nudorax", "whole head turned", ngeo)):
+            t = timed_k(lambda: hops.attn_prep(qkv, H * hd, (H + G) * hd, ge, freq, None, False, 1e-6, pos, seq, bt, kc, vc, q_norm=qw, k_norm=kw_, norm_whole=True))
+            add(fam, f"attn_prep (norm over all heads, {nm}, page write)", f"T={T_} H={H} G={G}", t, nb, 0, VALU_F32)
+        down, qq, proj, qn, qabs, cw = f32(T_, Rq + R + dr + H), f32(T_, hq), f32(T_, hq + R + dr), bf(T_, H * hd), f32(T_, H * dpad), bf(R)
+        nb = T_ * (hq * 4 + (R + dr) * 4 + H * hd * 2 + H * (dpad - R) * 4 + dpad * 2)
+        cache = lc.view(nblk, page, dpad)
+        t = timed_k(lambda: hops.latent_prep(down, Rq, lg, freq, 1.0, cw, 1e-6, pos, seq, bt, qn, qabs, cache, q=qq, layout=1))
+        add("kerotar", "latent_prep (queries of their own)", f"T={T_} H={H}", t, nb, 0, VALU_F32)
+        t = timed_k(lambda: hops.latent_prep(proj, hq, lg, freq, 1.2, cw, 1e-6, pos, seq, bt, qn, qabs, cache))
+        add("pokepel", "latent_prep", f"T={T_} H={H}", t, nb, 0, VALU_F32)
+        qlw, hn, hg, hw = bf(Rq), f32(T_, H * hd), f32(T_, H * hd), bf(H * hd)
+        t = timed_k(lambda: hops.head_norm(down[:, :Rq], 1, Rq, qlw, 1e-6))
+        add("kerotar", "norm of the query latent", f"T={T_} rank={Rq}", t, T_ * Rq * 6, 0, VALU_F32)
+        t = timed_k(lambda: hops.head_norm(hn, 1, H * hd, hw, 1e-6, hg, 0, gate_act="sigmoid"))
+        add("nudorax", "norm over all heads (weight, sigmoid gate)", f"T={T_} H={H} vdim={hd}", t, T_ * H * hd * 10, 0, VALU_F32)
+        wuk, wuv, ol, vg = bf(H, R, hd), bf(H, hd, R), bf(T_, H * R), f32(T_, H * hd)
+        t = timed_k(lambda: hops.dense_grouped(ol, wuv, x_step=R, y_step=hd))
+        add("kerotar", "dense_grouped heads (values)", f"M={T_} G={H} N={hd} K={R}", t, H * R * hd * 2 + T_ * H * (R * 2 + hd * 2), 2.0 * T_ * H * R * hd, MFMA_BF16)
+        t = timed_k(lambda: hops.dense_grouped(ol, wuv, x_step=R, y_step=hd, mul_sigmoid=vg))
+        add("pokepel", "dense_grouped heads (values x gate per channel)", f"M={T_} G={H} N={hd} K={R}", t, H * R * hd * 2 + T_ * H * (R * 2 + hd * 6), 2.0 * T_ * H * R * hd, MFMA_BF16)
+    for T_ in (prompt, 8, 1):
+        h, z = bf(T_, W), f32(T_, E) * 2
+        t = timed_k(lambda: hops.moe_route_sorted(z, E, 1, 1, top, chosen=True))
+        add("kerotar", "moe route + sort (softmax over the chosen)", f"T={T_} E={E} top={top}", t, T_ * (E * 4 + top * 16), 0, VALU_F32)
+        t = timed_k(lambda: hops.moe_route_sorted(z, E, gr["count"], gr["keep"], top))
+        add("pokepel", "moe route + sort (groups)", f"T={T_} E={E} top={top}", t, T_ * (E * 4 + top * 16), 0, VALU_F32)
+        ids, wts = hops.moe_route(z, 1, 1, top, chosen=True)
+        offs, src, place, tiles = hops.moe_align(ids, E)
+        n, used = T_ * top, len(set(ids.flatten().tolist()))
+        wgu, wdn, act = torch.stack([hops.group_gate_up(bf(fe, W), bf(fe, W)) for _ in range(E)]).contiguous(), bf(E, W, fe), bf(n, fe)
+        t = timed_k(lambda: hops.dense_grouped(h, wgu, offs=offs, gather=src, tiles=tiles, rows=n, gated=True, act=hops.ACT_SILU))
+        add("kerotar", "dense_grouped experts gated (Pokepel's too)", f"M={T_}x{top} E={E} ({used} used) N={2 * fe} K={W}", t, used * 2 * fe * W * 2 + n * (W + fe) * 2, 2.0 * n * 2 * fe * W, MFMA_BF16)
+        t = timed_k(lambda: hops.dense_grouped(act, wdn, offs=offs, tiles=tiles, rows=n, out_dtype=torch.float32))
+        add("kerotar", "dense_grouped experts down (Pokepel's too)", f"M={T_}x{top} E={E} ({used} used) N={W} K={fe}", t, used * fe * W * 2 + n * (fe * 2 + W * 4), 2.0 * n * fe * W, MFMA_BF16)
+        y, x, aa, bb, gt, extra, w1, pair = f32(n, W), f32(T_, W), f32(T_, W), f32(T_, W), f32(T_, 2 * W), f32(T_, W), bf(W), bf(T_, 2 * W)
+        nb = (n + 3 * T_) * W * 4 + T_ * W * 2
+        t = timed_k(lambda: hops.residual_norm(x, aa, hops.MoeSum(y, place, wts), 1.0, w1, None, 1e-6))
+        add("kerotar", "residual + mixture sum + norm", f"T={T_} top={top} W={W}", t, nb, 0, VALU_F32)
+        t = timed_k(lambda: hops.residual_round(x, aa, hops.MoeSum(y, place, wts), 1.0, pair[:, :W]))
+        add("kerotar", "residual + mixture sum, rounded (in front of a pass)", f"T={T_} top={top} W={W}", t, nb, 0, VALU_F32)
+        t = timed_k(lambda: hops.residual_norm(x, aa, hops.MoeSum(y, place, wts, extra), 1.0, w1, None, 1e-6, gate=gt))
+        add("pokepel", "gated residual + mixture sum + norm", f"T={T_} top={top} W={W}", t, nb + 3 * T_ * W * 4, 0, VALU_F32)
+        t = timed_k(lambda: hops.residual_norm(x, aa, bb, 1.0, w1, None, 1e-6))
+        add("kerotar", "residual + norm (fp32 stream)", f"M={T_} W={W}", t, stream_bytes(T_, W, 4, 1), 0, VALU_F32)
+        t = timed_k(lambda: hops.residual_norm(x, aa, bb, 1.0, w1, None, 1e-6, gate=gt))
+        add("pokepel", "gated residual + norm (fp32 stream)", f"M={T_} W={W}", t, stream_bytes(T_, W, 6, 1), 0, VALU_F32)
+        ids, table = torch.randint(0, s["vocab"], (T_,), device=dev, dtype=torch.int32), bf(s["vocab"], W)
+        t = timed_k(lambda: hops.embed_scaled(ids, table, 4.0, copy=pair[:, W:]))
+        add("kerotar", "embedding x scale (stream + rounded columns)", f"M={T_} W={W}", t, T_ * W * (2 + 4 + 2), 0, VALU_F32)
+        t = timed_k(lambda: hops.embed_scaled(ids, table, 8.0, rounded=True))
+        add("nudorax", "embedding x scale (stream + rounded copy)", f"M={T_} W={W}", t, T_ * W * (2 + 4 + 2), 0, VALU_F32)
+        # linears
+        lin = [("kerotar", "dense_linear in front of a pass [stream | embedding]", W, 2 * W, bf(W)), ("kerotar", "dense_linear q | k | v (window layer)", (H + 2 * G) * hd, W, None),
+               ("kerotar", "dense_linear dq | dkv | g | router (latent layer)", Rq + R + dr + H + E, W, None), ("kerotar", "dense_linear query up-projection", hq, Rq, None),
+               ("pokepel", "dense_linear q | dkv | g (latent layer)", hq + R + dr + H * hd, W, None)]
+        for fam, nm, N_, K_, bias in lin:
+            wi, xi = bf(N_, K_), bf(T_, K_)
+            t = timed_k(lambda: hops.dense_linear(xi, wi, bias, out_dtype=torch.float32))
+            add(fam, nm, f"M={T_} N={N_} K={K_}", t, N_ * K_ * 2 + T_ * (K_ * 2 + N_ * 4), 2.0 * T_ * N_ * K_, MFMA_BF16)
+        wg, wu = hops.group_gate_up(bf(ff // 32 * 32, W), bf(ff // 32 * 32, W)), bf(ff, W)
+        t = timed_k(lambda: hops.dense_linear(h, wg, gated=True, act=hops.ACT_SWIGLU_CLAMP, act_param=7.0))
+        add("kerotar", "dense_linear gate | up (clamped)", f"M={T_} N={wg.shape[0]} K={W}", t, wg.numel() * 2 + T_ * (W + ff) * 2, 2.0 * T_ * wg.numel(), MFMA_BF16)
+        t = timed_k(lambda: hops.dense_linear(h, wu, out_dtype=torch.float32))
+        add("pokepel", "dense_linear up (PolyNorm)", f"M={T_} N={ff} K={W}", t, wu.numel() * 2 + T_ * (W * 2 + ff * 4), 2.0 * T_ * wu.numel(), MFMA_BF16)
+    return rows
+
+
 def stream_bytes(T_, W, f32_streams, bf16_streams):
     return T_ * W * (4 * f32_streams + 2 * bf16_streams)
 
 
 KERNEL_TABLES = {"pokepel": (kernel_table_pokepel, "nufalorn"), "nepudra": (kernel_table_nepudra, "nufalorn"), "nudorax": (kernel_table_nudorax, "pokepel"),
-                 "dupenex": (kernel_table_dupenex, "nudorax")}
+                 "dupenex": (kernel_table_dupenex, "nudorax"), "kerotar": (kernel_table_kerotar, "pokepel")}
 
 
 def run_pokepel(args, dev, sizes, member="pokepel"):

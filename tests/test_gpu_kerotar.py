@@ -132,7 +132,7 @@ def test_latent_rows_with_queries_from_a_buffer_of_their_own(layout):
         assert float(cache[[1, 2]].abs().max()) == 0.0
 
 
-@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 32, 16), (2, 2, 128, 48), (4, 1, 64, 64), (3, 1, 20, 12), (1, 1, 256, 160)])
+@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 32, 16), (2, 2, 128, 48), (4, 1, 64, 64), (3, 1, 20, 12), (1, 1, 256, 160), (4, 1, 160, 32), (4, 2, 64, 192)])
 @pytest.mark.parametrize("window,keep", [(40, 20), (70, 0), (0, 9), (1, 1), (5, 64), (33, 65), (64, 31), (32, 32), (3, 33), (100, 400)])
 def test_window_with_kept_first_tokens(H, G, d, dv, window, keep):
     """Both attention kernels over scattered pages: a whole prompt, a portion in the middle, and rows far behind the kept tokens; with a sink and head gates."""
